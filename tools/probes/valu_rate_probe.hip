@@ -37,8 +37,6 @@ __global__ void __launch_bounds__(1024) probe(uint32_t* out, int iters, uint32_t
           float v;
           asm volatile("v_cvt_f32_ubyte0_e32 %0, %1" : "=v"(v) : "v"(src));
           r[i] = __builtin_bit_cast(uint32_t, v);
-        } else if constexpr (KIND == 2) {  // v_pk_fma_f32
-          asm volatile("v_pk_fma_f32 %0, %1, %2, %3" : "=v"(f[i]) : "v"(s2), "v"(c2), "v"(c2));
         } else if constexpr (KIND == 3) {  // v_cvt_pk_bf16_f32
           asm volatile("v_cvt_pk_bf16_f32 %0, %1, %2" : "=v"(r[i]) : "v"(scale), "v"(scale));
         } else if constexpr (KIND == 4) {  // v_perm_b32
@@ -125,7 +123,6 @@ int main(int argc, char** argv) {
     run<0>("v_cvt_scalef32_pk_bf16_fp8", w, d_out, n_cu, mhz);
     run<9>("v_cvt_scalef32_pk_bf16_fp8 op_sel hi", w, d_out, n_cu, mhz);
     run<1>("v_cvt_f32_ubyte0", w, d_out, n_cu, mhz);
-    run<2>("v_pk_fma_f32", w, d_out, n_cu, mhz);
     run<3>("v_cvt_pk_bf16_f32", w, d_out, n_cu, mhz);
     run<4>("v_perm_b32", w, d_out, n_cu, mhz);
     run<5>("v_and_b32", w, d_out, n_cu, mhz);
