@@ -11,8 +11,9 @@ import os
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "csrc", "libslm_hip.so")
+LATENT_LIB_PATH = os.path.join(_HERE, "csrc", "libslm_latent.so")
 
-SLM_F16, SLM_BF16 = 0, 1
+SLM_F16, SLM_BF16, SLM_F32 = 0, 1, 2   # (SLM_F32: libslm_latent only)
 SLM_W4_GPTQ, SLM_W4_AWQ = 0, 1
 SLM_W8_GPTQ, SLM_W8_AWQ = 2, 3  # 8-bit checkpoints: slm_w8_prepack_* (two int4 planes)
 SLM_W4_PAIRED = 0x10
@@ -204,3 +205,94 @@ def check(rc: int, what: str) -> None:
     if rc != 0:
         detail = f" [{lib().slm_last_hip_error().decode()}]" if rc == -4 else ""
         raise SlmError(f"{what} failed: {lib().slm_status_string(rc).decode()} ({rc}){detail}")
+
+
+# ---- libslm_latent.so (include/slm_latent.h) -------------------------------------------------------
+def _fields(*groups):
+    return [(n, t) for t, names in groups for n in names.split()]
+
+
+class ResidualNormArgs(C.Structure):
+    """slm_residual_norm_args."""
+    _fields_ = _fields((C.c_void_p, "resid delta slabs tokens positions embed pos_table row_index weight out"),
+                       (C.c_int64, "rows width ld_delta ld_embed ld_out slab_stride"),
+                       (C.c_float, "eps"), (C.c_int32, "n_slabs mode dtype"))
+
+
+RN_EMBED, RN_ADD, RN_SLABS, RN_PLAIN = range(4)
+
+
+class LinearArgs(C.Structure):
+    """slm_linear_args."""
+    _fields_ = _fields((C.c_void_p, "x w y gate"),
+                       (C.c_int64, "M N K ldx ldw ldy ld_gate x_batch w_batch y_batch"),
+                       (C.c_float, "alpha limit glu_alpha"), (C.c_int32, "batch n_splits epilogue dtype"))
+
+
+LIN_STORE, LIN_F32, LIN_SLABS, LIN_GLU, LIN_GATE = range(5)
+
+
+class LatentAppendArgs(C.Structure):
+    """slm_latent_append_args."""
+    _fields_ = _fields((C.c_void_p, "proj cache q_abs norm_weight cos_sin positions slots"),
+                       (C.c_int64, "rows abs_rows ld_proj off_c off_r max_positions"),
+                       (C.c_int32, "heads q_dim q_rot rank rot c_pad r_pad dtype"), (C.c_float, "eps"))
+
+
+class LatentAttnArgs(C.Structure):
+    """slm_latent_attn_args."""
+    _fields_ = _fields((C.c_void_p, "q_abs cache out positions q_cu block_table block_cu workspace"),
+                       (C.c_size_t, "workspace_bytes"), (C.c_int64, "rows"),
+                       (C.c_int32, "batch heads c_pad r_pad block_size window max_kv_len n_splits"),
+                       (C.c_float, "scale"), (C.c_int32, "dtype generic"))
+
+
+class LatentPrefillArgs(C.Structure):
+    """slm_latent_prefill_args."""
+    _fields_ = _fields((C.c_void_p, "q ctx kv gate out tiles"),
+                       (C.c_int64, "ld_q ld_out n_rows n_ctx gate_off"),
+                       (C.c_int32, "n_tiles heads q_dim c_pad r_pad v_pad window"), (C.c_float, "scale"))
+
+
+LATENT_Q_TILE = 128
+
+_latent = None
+
+
+def latent_lib() -> C.CDLL:
+    """Load libslm_latent.so or raise -- never falls back."""
+    global _latent
+    if _latent is not None:
+        return _latent
+    if not os.path.exists(LATENT_LIB_PATH):
+        raise SlmError(f"{LATENT_LIB_PATH} not found: build it with `python -m scalellm_amd.build --library latent`")
+    import torch  # noqa: F401  (one HIP runtime per process: see lib())
+    L = C.CDLL(LATENT_LIB_PATH)
+    i32, i64, f32, ptr, P = C.c_int32, C.c_int64, C.c_float, C.c_void_p, C.POINTER
+    for name, restype, argtypes in [
+        ("slm_latent_version", C.c_char_p, []),
+        ("slm_latent_status_string", C.c_char_p, [C.c_int]),
+        ("slm_latent_last_hip_error", C.c_char_p, []),
+        ("slm_residual_norm", C.c_int, [P(ResidualNormArgs), ptr]),
+        ("slm_linear", C.c_int, [P(LinearArgs), ptr]),
+        ("slm_clamped_glu", C.c_int, [ptr, ptr, i64, i64, i64, i64, f32, f32, i32, ptr]),
+        ("slm_latent_append", C.c_int, [P(LatentAppendArgs), ptr]),
+        ("slm_latent_attn_workspace_bytes", C.c_size_t, [P(LatentAttnArgs)]),
+        ("slm_latent_attn", C.c_int, [P(LatentAttnArgs), ptr]),
+        ("slm_latent_attn_is_mfma", C.c_int, [i32, i32, i32]),
+        ("slm_latent_gather", C.c_int, [ptr, ptr, ptr, i64, i64, ptr]),
+        ("slm_latent_prefill", C.c_int, [P(LatentPrefillArgs), ptr]),
+        ("slm_latent_prefill_supported", C.c_int, [i32, i32, i32]),
+    ]:
+        fn = getattr(L, name)
+        fn.restype = restype
+        fn.argtypes = argtypes
+    _latent = L
+    return L
+
+
+def latent_check(rc: int, what: str) -> None:
+    if rc != 0:
+        L = latent_lib()
+        detail = f" [{L.slm_latent_last_hip_error().decode()}]" if rc == -4 else ""
+        raise SlmError(f"{what} failed: {L.slm_latent_status_string(rc).decode()} ({rc}){detail}")

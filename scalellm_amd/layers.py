@@ -19,14 +19,23 @@ the reference so parity tests read like the reference's own layer tests.
 """
 from __future__ import annotations
 
-from dataclasses import dataclass
-from typing import Dict, Optional, Tuple
+from dataclasses import dataclass, field
+from typing import Dict, Optional, Sequence, Tuple
 
 import torch
 
 from . import kernels
 from .model_parallel import (ParallelArgs, gather_from_model_parallel_region,
                              reduce_from_model_parallel_region)
+
+
+@dataclass
+class Portion:
+    """A sequence of the step that brings several tokens (a prompt or a part of one), as the HOST knows it."""
+    row0: int      # its first row in the step
+    q_len: int
+    kv_len: int    # tokens in the cache after the step
+    blocks: object  # numpy int32: first-slot ids of its blocks
 
 
 @dataclass
@@ -45,6 +54,15 @@ class InputParameters:
     # SIZES where they settle it (uniform_kv_hint below -- what an unchanged engine gets); < 0 = known NOT to
     # be uniform (no derivation: a graph captured over padded static buffers, the half of a ragged batch)
     kv_total_len: int = 0
+    # extension: rows of the step whose logits are wanted (int32; the reference's selected token indexes of
+    # SamplingParameters).  None = the last row of every sequence
+    logit_rows: Optional[torch.Tensor] = None
+    # extension: the sequences at the END of the step that bring whole portions, for models with a kernel of their
+    # own for them (the rows in front of the first portion are single tokens).  Empty = nothing known: every row
+    # is served on its own
+    portions: Sequence[Portion] = ()
+    # what a model derived from `portions` for this step (one entry per attention window)
+    plans: Dict[object, object] = field(default_factory=dict)
 
 
 def uniform_kv_hint(kv_total_len: int, n_seqs: int, q_max_seq_len: int, kv_max_seq_len: int,
