@@ -48,9 +48,9 @@ template <typename T>
 __device__ __forceinline__ uint32_t pack2(float a, float b);
 template <>
 __device__ __forceinline__ uint32_t pack2<bf16_tag>(float a, float b) {
-  uint32_t r;
-  asm("v_cvt_pk_bf16_f32 %0, %1, %2" : "=v"(r) : "v"(a), "v"(b));
-  return r;
+  // (v_cvt_pk_bf16_f32, left to the compiler: behind an asm statement it inserts no wait states, and an MFMA that
+  //  reads the result within two of them gets the old register)
+  return __builtin_bit_cast(uint32_t, __builtin_convertvector((f32x2{a, b}), bf16x2_t));
 }
 template <>
 __device__ __forceinline__ uint32_t pack2<f16_tag>(float a, float b) {
@@ -201,8 +201,13 @@ __device__ __forceinline__ u32x4 rms_apply8(const float (&h)[8], const float rs,
   float o[8];
 #pragma unroll
   for (int j = 0; j < 8; ++j) {
-    const float n16 = lo_f32<T>((uint32_t)pack1<T>(h[j] * rs));
+    // both products are fp32 values in a register before they are rounded to T (see silu_mul1: folding
+    // "multiply, then round to fp16" into one instruction in some callers only would change bits)
+    float n = h[j] * rs;
+    asm("" : "+v"(n));
+    const float n16 = lo_f32<T>((uint32_t)pack1<T>(n));
     o[j] = n16 * wf[j];
+    asm("" : "+v"(o[j]));
   }
   u32x4 r;
   r.x = pack2<T>(o[0], o[1]); r.y = pack2<T>(o[2], o[3]);
