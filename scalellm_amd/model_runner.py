@@ -194,7 +194,8 @@ class ModelRunner:
     def forward(self, tokens, positions, params: InputParameters, num_sequences: Optional[int] = None):
         bs = int(params.q_cu_seq_lens.numel() - 1) if num_sequences is None else num_sequences
         g = self.graphs.get(bs)
-        if g is not None:
+        # (a graph gives the last row of every sequence: other rows are an eager step's)
+        if g is not None and getattr(params, "logit_rows", None) is None:
             nd = self.options.num_decoding_tokens
             if (params.kv_max_seq_len <= self.options.cuda_graph_max_seq_len and
                     params.q_max_seq_len == nd and tokens.numel() == bs * nd):
