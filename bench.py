@@ -484,11 +484,13 @@ def main():
     if "--probe-xgmi-ar" in sys.argv:
         _probe_xgmi_main()
         return
-    if "--model" in sys.argv and sys.argv[sys.argv.index("--model") + 1:][:1] == ["dagupel"]:
-        # the latent-attention design beside the Llama step at equal size: lines of its own (tools/bench_dagupel.py)
+    pre = argparse.ArgumentParser(add_help=False, allow_abbrev=False)
+    pre.add_argument("--model")
+    known, rest = pre.parse_known_args()
+    if known.model == "dagupel":
+        # the latent-attention design beside the Llama step at equal size: lines of its own
         from tools.bench_dagupel import main as bench_dagupel
-        at = sys.argv.index("--model")
-        raise SystemExit(bench_dagupel(sys.argv[1:at] + sys.argv[at + 2:]))
+        raise SystemExit(bench_dagupel(rest))
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=10)

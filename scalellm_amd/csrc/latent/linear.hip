@@ -169,13 +169,21 @@ static int lin_launch(const slm_linear_args& a, hipStream_t st) {
   linear_kernel<E, MT, NT, U, EPI><<<dim3((unsigned)gx, (unsigned)gy, (unsigned)gz), dim3(256), 0, st>>>(a);
   return hip_check_launch();
 }
+// Tiles by row count: one row block streams W with many steps in flight; with more rows the reads of x weigh as much
+// as those of W, and wider column blocks (where enough of them are left to fill the chip) read x less often.
 template <typename E, int EPI>
 static int lin_shape(const slm_linear_args& a, hipStream_t st) {
-  constexpr bool F32 = sizeof(E) == 4;
   constexpr int P = EPI == SLM_LIN_GLU ? 2 : 1;
-  if (a.M <= 16) return lin_launch<E, 1, P, F32 ? 1 : 4 / P, EPI>(a, st);
-  if (a.M <= 32 || F32) return lin_launch<E, 2, 2, F32 ? 1 : 2, EPI>(a, st);
-  return lin_launch<E, 4, 2, 2, EPI>(a, st);
+  if constexpr (sizeof(E) == 4) {
+    if (a.M <= 16) return lin_launch<E, 1, P, 1, EPI>(a, st);
+    return lin_launch<E, 2, 2, 1, EPI>(a, st);
+  } else {
+    if (a.M <= 4) return lin_launch<E, 1, P, 8 / P, EPI>(a, st);
+    if (a.M <= 16) return lin_launch<E, 1, P, 4 / P, EPI>(a, st);
+    const bool wide = a.N / 64 * a.batch * a.n_splits >= 256;
+    if (a.M <= 32) return wide ? lin_launch<E, 2, 4, 1, EPI>(a, st) : lin_launch<E, 2, 2, 2, EPI>(a, st);
+    return wide ? lin_launch<E, 4, 4, 1, EPI>(a, st) : lin_launch<E, 4, 2, 2, EPI>(a, st);
+  }
 }
 template <typename E>
 static int lin_epi(const slm_linear_args& a, hipStream_t st) {

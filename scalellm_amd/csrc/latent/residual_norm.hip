@@ -48,15 +48,21 @@ __global__ void __launch_bounds__(RN_THREADS) residual_norm_kernel(const slm_res
           for (int j = 0; j < V; ++j) x[s][j] += t[j];
         }
         if constexpr (MODE == SLM_RN_SLABS) {
+          // (all slab loads of a chunk in flight at once)
+          const float* sp = a.slabs + row * a.ld_delta + i;
           float d[V];
 #pragma unroll
           for (int j = 0; j < V; ++j) d[j] = 0.f;
-          const float* sp = a.slabs + row * a.ld_delta + i;
-          for (int k = 0; k < a.n_slabs; ++k) {
-            float t[V];
-            load_f32<V>(sp + k * a.slab_stride, t);
+          for (int k0 = 0; k0 < a.n_slabs; k0 += 8) {
+            float t[8][V];
 #pragma unroll
-            for (int j = 0; j < V; ++j) d[j] += t[j];
+            for (int k = 0; k < 8; ++k)
+              if (k0 + k < a.n_slabs) load_f32<V>(sp + (k0 + k) * a.slab_stride, t[k]);
+#pragma unroll
+            for (int k = 0; k < 8; ++k)
+              if (k0 + k < a.n_slabs)
+#pragma unroll
+                for (int j = 0; j < V; ++j) d[j] += t[k][j];
           }
 #pragma unroll
           for (int j = 0; j < V; ++j) x[s][j] += d[j];

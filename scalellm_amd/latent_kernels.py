@@ -15,7 +15,7 @@ from ._lib import SLM_BF16, SLM_F32, SlmError, latent_check
 from .kernels import reserve_workspace
 
 # rows up to which the weight-streaming kernel serves a bf16 product; above it the vendor GEMM does
-STREAM_MAX_ROWS = 64
+STREAM_MAX_ROWS = 32
 # clamped GLU: y = g * sigmoid(alpha * g) * (u + 1)
 GLU_ALPHA = 1.702
 

@@ -236,6 +236,27 @@ def test_graph_replays_equal_eager_steps():
     assert row_errors(outs[1], outs[0].astype(np.float64)).max() < 1e-2
 
 
+def test_graph_replays_of_a_batch_the_vendor_products_serve():
+    """40 decode rows: the projections are library products inside the graph; every replay equals the eager step."""
+    cfg, t, _, _ = _model("wide")
+    rng = np.random.default_rng(2)
+    prompts = [rng.integers(0, cfg["vocab"], 20 + k).tolist() for k in range(40)]
+    outs = []
+    for graphs in ([], [40]):
+        engine = _engine(cfg, t, torch.bfloat16, n_blocks=200, block_size=16, graph_batch_sizes=graphs, graph_max_seq_len=128)
+        engine.capture_graphs()
+        seqs = [_seq(k, p) for k, p in enumerate(prompts)]
+        _run(engine, [(s, len(s.tokens) - 9) for s in seqs])
+        rows = []
+        for k in range(9):
+            rows.append(engine.run_entries([(s, 1) for s in seqs])[1].float().cpu().numpy())
+            if k % 3 == 1:
+                _run(engine, [(_seq("x", prompts[3]), 5)])
+        outs.append(np.concatenate(rows))
+        assert engine.runner.num_graph_replayed == (9 if graphs else 0)
+    assert row_errors(outs[1], outs[0].astype(np.float64)).max() < 1e-2
+
+
 def test_preempted_sequences_start_over():
     cfg, t, _, _ = _model("tiny")
     from scalellm_amd.sampling import SamplingParams

@@ -82,7 +82,8 @@ def test_eps_is_inside_the_root():
 # ---- products ----------------------------------------------------------------------------------
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("M,N,K", [(1, 16, 64), (3, 48, 320), (16, 80, 1024), (17, 112, 192), (33, 96, 2048), (64, 272, 128),
-                                   (65, 64, 64), (200, 144, 256), (1, 4096, 4096)])
+                                   (65, 64, 64), (200, 144, 256), (1, 4096, 4096),
+                                   (30, 16416, 128), (20, 4096, 8192), (50, 16416, 64)])
 def test_linear_epilogues(M, N, K, dtype):
     lk = _lk()
     x, w = _rnd(1, M, K, dtype=dtype), _rnd(2, N, K, dtype=dtype, std=K ** -0.5)
