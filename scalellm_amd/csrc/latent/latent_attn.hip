@@ -7,8 +7,8 @@
 //
 // latent_attn_kernel (bf16, MFMA 16x16x32), eight waves, 32 cache rows per tile, a ring of four to eight tiles in LDS:
 //   staging   global -> LDS by LDS-DMA (a wave instruction writes 1 KiB linearly), all but one tile of the ring in flight
-//             behind counted waits; block-table entries of the whole range are staged in LDS first, so no other load
-//             sits in the vmcnt queue.  The image is swizzled on the source side: 16-byte unit u of row r holds chunk
+//             behind counted waits; block-table entries of the range are staged in LDS first (LA_TBL at a time), so
+//             no other load sits in the vmcnt queue.  The image is swizzled on the source side: 16-byte unit u of row r holds chunk
 //             u ^ (r / 2 % 8), which keeps both fragment reads below off each other's banks
 //   S = C Q^T 16 x 16 blocks, one a wave (16 heads: half a contraction each), A = cache rows, B = the wave's head
 //             block, held in registers; S to LDS.  One tile AHEAD of the rest, so that a tile costs one barrier and a
@@ -58,7 +58,7 @@ __device__ __forceinline__ void wait_tiles(int tiles) {
 }
 
 constexpr int LA_KT = 32;     // cache rows per tile
-constexpr int LA_TBL = 1024;  // block-table entries staged in LDS (longer ranges look them up in memory)
+constexpr int LA_TBL = 1024;  // block-table entries staged in LDS at a time
 
 template <int KP, int RP, int MH>
 __global__ void __launch_bounds__(512) latent_attn_kernel(const LatentAttnK p) {
@@ -124,17 +124,13 @@ __global__ void __launch_bounds__(512) latent_attn_kernel(const LatentAttnK p) {
     lo = min(hi, lo + split * per);
     hi = min(hi, lo + per);
   }
-  const int n_tiles = (hi - lo + KT - 1) / KT;
-  const int blk0 = lo >> p.block_shift;
-  const int n_ent = n_tiles > 0 ? ((hi - 1) >> p.block_shift) - blk0 + 1 : 0;
-  const bool staged = n_ent <= LA_TBL;
-  if (staged)
-    for (int i = tid; i < n_ent; i += 512) tbl[i] = a.block_table[bcu + blk0 + i];
   // (the queries have arrived before the first DMA is issued: a wait for them later would drain the ring)
 #pragma unroll
   for (int s = 0; s < QW; ++s) asm volatile("" : "+v"(qf[s]));
-  __syncthreads();
 
+  // the segment of the range whose block-table entries are staged: keys [lo, hi)
+  const int range_hi = hi;
+  int blk0 = 0, n_tiles = 0;
   const uint32_t ring0 = (uint32_t)(uintptr_t)(__attribute__((address_space(3))) char*)ring;
   const char* cache = reinterpret_cast<const char*>(a.cache);
   // (inline asm: through the builtin the compiler makes every read of the ring wait for the DMA into its other tiles)
@@ -146,11 +142,7 @@ __global__ void __launch_bounds__(512) latent_attn_kernel(const LatentAttnK p) {
       const int u = min(wave + 8 * i, NTOT - 1) * 64 + lane;
       const int r = u / CHP, c = min((u % CHP) ^ ((r >> 1) & 7), CH - 1);
       const int key = min(lo + t * KT + r, hi - 1);  // rows past the end re-read the last one; masked below
-      const int blk = key >> p.block_shift;
-      // (address spaces spelled out: merged into one flat load the look-up would wait for the whole ring)
-      int slot;
-      if (staged) slot = ((__attribute__((address_space(3))) const int*)tbl)[blk - blk0];
-      else slot = ((__attribute__((address_space(1))) const int*)a.block_table)[bcu + blk];
+      const int slot = tbl[(key >> p.block_shift) - blk0];
       src[i] = cache + (int64_t)(slot + (key & p.block_mask)) * (R * 2) + 16 * c;
     }
 #pragma unroll
@@ -172,10 +164,6 @@ __global__ void __launch_bounds__(512) latent_attn_kernel(const LatentAttnK p) {
     for (int t = 0; t < NT; ++t) o[m][t] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
 
-#pragma unroll
-  for (int t = 0; t < NBUF - 1; ++t)
-    if (t < n_tiles) issue(t);
-
   // fragment reads: A of the scores (row l16 of a 16-key block, chunk 4 i + g), and the transpose read (keys
   // 8 g + l16 / 4 and + 4, 8-byte piece l16 % 4 of a 16-column block)
   const uint32_t k_row = (uint32_t)l16 * ROWB, k_x = (uint32_t)((l16 >> 1) & 7) ^ (uint32_t)g;
@@ -185,22 +173,26 @@ __global__ void __launch_bounds__(512) latent_attn_kernel(const LatentAttnK p) {
   const uint32_t tr_c = (uint32_t)wave * (2 * NT);
   const bool columns = KP >= 128 || wave < KP / 16;
 
-  bf16x8_t kf[QW];
-  auto read_rows = [&](int t) {   // A fragments of tile t
+  constexpr int QC = QW > 10 ? (QW + 1) / 2 : QW;   // k-steps read ahead of the products (register budget)
+  bf16x8_t kf[QC];
+  auto read_rows = [&](int t, int first) {   // A fragments of tile t, k-steps from `first` of this wave's
     const uint32_t base = ring0 + (uint32_t)(t % NBUF) * TILE + (uint32_t)(16 * kb) * ROWB + k_row;
 #pragma unroll
-    for (int i = 0; i < QW; ++i) {
-      const uint32_t step = (uint32_t)(kh * QW + i);
-      kf[i] = *(__attribute__((address_space(3))) const bf16x8_t*)(uintptr_t)(
-          base + (((4u * (KH * QW != QS ? min(step, (uint32_t)QS - 1) : step)) ^ k_x) << 4));
+    for (int i = 0; i < QC; ++i) {
+      const uint32_t step = (uint32_t)(kh * QW + first + i);
+      kf[i] = *(__attribute__((address_space(3))) const bf16x8_t*)(uintptr_t)(base + (((4u * min(step, (uint32_t)QS - 1)) ^ k_x) << 4));
     }
   };
   auto score = [&](int t) {
     f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int i = 0; i < QW; i += 2) {
-      s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[i], qf[i], s0, 0, 0, 0);
-      if (i + 1 < QW) s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[i + 1], qf[i + 1], s1, 0, 0, 0);
+    for (int c = 0; c < QW; c += QC) {
+      if (c > 0) read_rows(t, c);
+#pragma unroll
+      for (int i = 0; i < QC; i += 2) {
+        if (c + i < QW) s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[i], qf[c + i], s0, 0, 0, 0);
+        if (i + 1 < QC && c + i + 1 < QW) s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[i + 1], qf[c + i + 1], s1, 0, 0, 0);
+      }
     }
     // lane: head l16, keys 16 kb + 4 g .. + 3
     *reinterpret_cast<f32x4*>(&sc[t & 1][(16 * (MH * kh + hw) + l16) * SS + 16 * kb + 4 * g]) = s0 + s1;
@@ -209,116 +201,133 @@ __global__ void __launch_bounds__(512) latent_attn_kernel(const LatentAttnK p) {
     if (NTOT % 8 == 0 || wave < NTOT % 8) wait_tiles<NBUF - 2, NHI>(younger);
     else wait_tiles<NBUF - 2, NLO>(younger);
   };
-  if (n_tiles > 0) {
+  for (; lo < range_hi; lo = hi) {
+    blk0 = lo >> p.block_shift;
+    hi = min(range_hi, (blk0 + LA_TBL) << p.block_shift);
+    n_tiles = (hi - lo + KT - 1) / KT;
+    for (int i = tid; i <= ((hi - 1) >> p.block_shift) - blk0; i += 512) tbl[i] = a.block_table[bcu + blk0 + i];
+    __syncthreads();
+#pragma unroll 1
+    for (int t = 0; t < min(NBUF - 1, n_tiles); ++t) issue(t);
     arrived(min(NBUF - 2, n_tiles - 1));
     lds_barrier();
     if (scorer) {
-      read_rows(0);
+      read_rows(0, 0);
       score(0);
     }
-  }
-  for (int t = 0; t < n_tiles; ++t) {
-    const int k0 = lo + t * KT;
-    if (t + 1 < n_tiles) arrived(min(NBUF - 3, n_tiles - 2 - t));
-    lds_barrier();   // tile t + 1 and the scores of tile t are there, tile t - 1 is done with
-    if (t + NBUF - 1 < n_tiles) issue(t + NBUF - 1);
-    const uint32_t tile = ring0 + (uint32_t)(t % NBUF) * TILE;
-    const bool next = scorer && t + 1 < n_tiles;
-    if (next) read_rows(t + 1);
-    if (!columns) {   // (a latent of 64: four waves hold all of it)
-      if (next) score(t + 1);
-      continue;
-    }
-    // ---- scores back in the B layout of the second product, C^T fragments behind them (read under the soft-max)
-    f32x4 raw[MH][KH][2];
-#pragma unroll
-    for (int m = 0; m < MH; ++m)
-#pragma unroll
-      for (int k = 0; k < KH; ++k) {
-        const float* sp = &sc[t & 1][(16 * (MH * k + m) + l16) * SS + 8 * g];
-        raw[m][k][0] = *reinterpret_cast<const f32x4*>(sp);
-        raw[m][k][1] = *reinterpret_cast<const f32x4*>(sp + 4);
+    for (int t = 0; t < n_tiles; ++t) {
+      const int k0 = lo + t * KT;
+      if (t + 1 < n_tiles) arrived(min(NBUF - 3, n_tiles - 2 - t));
+      lds_barrier();   // tile t + 1 and the scores of tile t are there, tile t - 1 is done with
+      if (t + NBUF - 1 < n_tiles) issue(t + NBUF - 1);
+      const uint32_t tile = ring0 + (uint32_t)(t % NBUF) * TILE;
+      const bool next = scorer && t + 1 < n_tiles;
+      if (next) read_rows(t + 1, 0);
+      if (!columns) {   // (a latent of 64: four waves hold all of it)
+        if (next) score(t + 1);
+        continue;
       }
-    __builtin_amdgcn_sched_barrier(0);
-    tr_v8 ct[NT];
-#pragma unroll
-    for (int t2 = 0; t2 < NT; ++t2) {
-      const uint32_t cc = tr_c + 2u * t2, ad = tile + tr_row;
-      const tr_v4 c0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((tr_lds_v4*)(uintptr_t)(ad + ((cc ^ tr_x0) << 4)));
-      const tr_v4 c1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((tr_lds_v4*)(uintptr_t)(ad + 4 * ROWB + ((cc ^ tr_x1) << 4)));
-      ct[t2] = __builtin_shufflevector(c0, c1, 0, 1, 2, 3, 4, 5, 6, 7);
-    }
-    __builtin_amdgcn_sched_barrier(0);
-    if (next) score(t + 1);
-    // ---- soft-max
-    bf16x8_t pf[MH];
-#pragma unroll
-    for (int m = 0; m < MH; ++m) {
-      float v[8];
-      float mx = M_INIT_F;
-#pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        float x = raw[m][0][j >> 2][j & 3];
-#pragma unroll
-        for (int k = 1; k < KH; ++k) x += raw[m][k][j >> 2][j & 3];
-        v[j] = k0 + 8 * g + j < hi ? x * p.scale2 : -INFINITY;
-        mx = fmaxf(mx, v[j]);
-      }
-      mx = max_over_groups(mx);
-      const float m_new = fmaxf(m_run[m], mx);
-      const float alpha = fast_exp2(m_run[m] - m_new);
-      m_run[m] = m_new;
-      float sum = 0.f;
-      u32x4 w;
-#pragma unroll
-      for (int j = 0; j < 8; j += 2) {
-        const float e0 = fast_exp2(v[j] - m_new), e1 = fast_exp2(v[j + 1] - m_new);
-        sum += e0 + e1;
-        w[j >> 1] = pack2<bf16_tag>(e0, e1);
-      }
-      pf[m] = __builtin_bit_cast(bf16x8_t, w);
-      l_run[m] = l_run[m] * alpha + sum;
-      if (__any(alpha != 1.0f)) {
-#pragma unroll
-        for (int t2 = 0; t2 < NT; ++t2) o[m][t2] *= alpha;
-      }
-    }
-    // ---- O^T += C^T P^T
-#pragma unroll
-    for (int t2 = 0; t2 < NT; ++t2)
+      // ---- scores back in the B layout of the second product, C^T fragments behind them (read under the soft-max)
+      f32x4 raw[MH][KH][2];
 #pragma unroll
       for (int m = 0; m < MH; ++m)
-        o[m][t2] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, ct[t2]), pf[m], o[m][t2], 0, 0, 0);
+#pragma unroll
+        for (int k = 0; k < KH; ++k) {
+          const float* sp = &sc[t & 1][(16 * (MH * k + m) + l16) * SS + 8 * g];
+          raw[m][k][0] = *reinterpret_cast<const f32x4*>(sp);
+          raw[m][k][1] = *reinterpret_cast<const f32x4*>(sp + 4);
+        }
+      __builtin_amdgcn_sched_barrier(0);
+      tr_v8 ct[NT];
+#pragma unroll
+      for (int t2 = 0; t2 < NT; ++t2) {
+        const uint32_t cc = tr_c + 2u * t2, ad = tile + tr_row;
+        const tr_v4 c0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((tr_lds_v4*)(uintptr_t)(ad + ((cc ^ tr_x0) << 4)));
+        const tr_v4 c1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((tr_lds_v4*)(uintptr_t)(ad + 4 * ROWB + ((cc ^ tr_x1) << 4)));
+        ct[t2] = __builtin_shufflevector(c0, c1, 0, 1, 2, 3, 4, 5, 6, 7);
+      }
+      __builtin_amdgcn_sched_barrier(0);
+      if (next) score(t + 1);
+      // ---- soft-max
+      bf16x8_t pf[MH];
+#pragma unroll
+      for (int m = 0; m < MH; ++m) {
+        float v[8];
+        float mx = M_INIT_F;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+          float x = raw[m][0][j >> 2][j & 3];
+#pragma unroll
+          for (int k = 1; k < KH; ++k) x += raw[m][k][j >> 2][j & 3];
+          v[j] = k0 + 8 * g + j < hi ? x * p.scale2 : -INFINITY;
+          mx = fmaxf(mx, v[j]);
+        }
+        mx = max_over_groups(mx);
+        const float m_new = fmaxf(m_run[m], mx);
+        const float alpha = fast_exp2(m_run[m] - m_new);
+        m_run[m] = m_new;
+        float sum = 0.f;
+        u32x4 w;
+#pragma unroll
+        for (int j = 0; j < 8; j += 2) {
+          const float e0 = fast_exp2(v[j] - m_new), e1 = fast_exp2(v[j + 1] - m_new);
+          sum += e0 + e1;
+          w[j >> 1] = pack2<bf16_tag>(e0, e1);
+        }
+        pf[m] = __builtin_bit_cast(bf16x8_t, w);
+        l_run[m] = l_run[m] * alpha + sum;
+        if (__any(alpha != 1.0f)) {
+#pragma unroll
+          for (int t2 = 0; t2 < NT; ++t2) o[m][t2] *= alpha;
+        }
+      }
+      // ---- O^T += C^T P^T
+#pragma unroll
+      for (int t2 = 0; t2 < NT; ++t2)
+#pragma unroll
+        for (int m = 0; m < MH; ++m)
+          o[m][t2] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, ct[t2]), pf[m], o[m][t2], 0, 0, 0);
+    }
+    lds_barrier();   // ring and table are free for the next segment
   }
-  if (!columns) return;
 
-  // lane: head l16 of block m, latent columns 16 NT wave + 16 t + 4 g .. + 3
+  // The accumulators (lane: head l16 of block m, latent columns 16 NT wave + 16 t + 4 g .. + 3) go through the ring, so
+  // that whole lines leave the chip: straight from the registers a store touches 64 bytes of 16 rows.
+  constexpr int OS = KP + 4;   // row stride (floats)
+  static_assert(16 * MH * OS * 4 <= NBUF * TILE, "the output tile fits the ring");
+  float* ot = reinterpret_cast<float*>(ring);
 #pragma unroll
   for (int m = 0; m < MH; ++m) {
+    if (columns) {
+#pragma unroll
+      for (int t = 0; t < NT; ++t) *reinterpret_cast<f32x4*>(ot + (16 * m + l16) * OS + wave * (16 * NT) + 16 * t + 4 * g) = o[m][t];
+    }
     float l = l_run[m];
     l += __shfl_xor(l, 16, 64);
     l += __shfl_xor(l, 32, 64);
-    const int h = h0 + 16 * m + l16;
-    if (h >= a.heads) continue;
-    const int64_t rh = row * a.heads + h;
-    const int c0 = wave * (16 * NT) + 4 * g;
-    if (p.n_splits == 1) {
-      const float inv = 1.0f / l;  // (every row sees itself: l > 0)
-      bf16* out = reinterpret_cast<bf16*>(a.out) + rh * KP + c0;
-#pragma unroll
-      for (int t = 0; t < NT; ++t)
-        *reinterpret_cast<u32x2*>(out + 16 * t) = u32x2{pack2<bf16_tag>(o[m][t].x * inv, o[m][t].y * inv),
-                                                        pack2<bf16_tag>(o[m][t].z * inv, o[m][t].w * inv)};
-    } else {
-      const int64_t pi = rh * p.n_splits + split;
-      float* out = p.o_part + pi * KP + c0;
-#pragma unroll
-      for (int t = 0; t < NT; ++t) *reinterpret_cast<f32x4*>(out + 16 * t) = o[m][t];
-      if (wave == 0 && g == 0) {
-        p.ml_part[2 * pi] = m_run[m];
-        p.ml_part[2 * pi + 1] = l;
-      }
+    if (wave == 0 && g == 0) {
+      sc[0][16 * m + l16] = m_run[m];
+      sc[1][16 * m + l16] = l;
     }
+  }
+  __syncthreads();
+  const int n_heads = min(16 * MH, a.heads - h0);
+  for (int i = tid; i < n_heads * (KP / 4); i += 512) {
+    const int hr = i / (KP / 4), c = i % (KP / 4) * 4;
+    const int64_t rh = row * a.heads + h0 + hr;
+    f32x4 v = *reinterpret_cast<const f32x4*>(ot + hr * OS + c);
+    if (p.n_splits == 1) {
+      v *= 1.0f / sc[1][hr];  // (every row sees itself: the sum is positive)
+      *reinterpret_cast<u32x2*>(reinterpret_cast<bf16*>(a.out) + rh * KP + c) =
+          u32x2{pack2<bf16_tag>(v.x, v.y), pack2<bf16_tag>(v.z, v.w)};
+    } else {
+      *reinterpret_cast<f32x4*>(p.o_part + (rh * p.n_splits + split) * KP + c) = v;
+    }
+  }
+  if (p.n_splits > 1 && tid < n_heads) {
+    const int64_t pi = (row * a.heads + h0 + tid) * p.n_splits + split;
+    p.ml_part[2 * pi] = sc[0][tid];
+    p.ml_part[2 * pi + 1] = sc[1][tid];
   }
 }
 

@@ -137,7 +137,7 @@ def test_clamped_glu_bends_where_it_should(dtype):
 
 # ---- rotation, latent norm, cache --------------------------------------------------------------
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("heads,q_dim,rot,rank", [(1, 32, 2, 5), (3, 64, 32, 64), (20, 96, 34, 100), (2, 32, 64, 500)])
+@pytest.mark.parametrize("heads,q_dim,rot,rank", [(1, 32, 2, 5), (3, 64, 32, 80), (20, 96, 34, 100), (2, 32, 64, 500)])
 def test_append_norms_rotates_and_writes_its_slots(heads, q_dim, rot, rank, dtype):
     from scalellm_amd.latent_layers import YarnScaling, round_up, rotary_table
     lk, eps, rows = _lk(), 1e-4, 7
@@ -253,8 +253,23 @@ def test_latent_attention_sees_exactly_its_window(dtype):
                     assert (float(out[i].float()[:, :8].min()) > 8.5) == seen, (block, window, p)
 
 
+@pytest.mark.parametrize("block,lens", [(1, [2500, 1023, 1024, 1025]), (2, [5000, 2049])])
+def test_latent_attention_of_more_blocks_than_are_staged_at_once(block, lens):
+    lk, c_pad, r_pad, H, dt = _lk(), 64, 32, 3, torch.bfloat16
+    pg = Paged(lens, block, c_pad, r_pad, dt)
+    q = _rnd(1, len(lens), H, c_pad + r_pad, dtype=dt)
+    pos = pg.dev([n - 1 for n in lens])
+    for window in (0, 1500):
+        want = np.stack([_attn_ref(_f64(q[i]), pg.rows(i), n - 1, window, 0.2, c_pad) for i, n in enumerate(lens)])
+        for splits in (1, 2):
+            out = torch.empty(len(lens), H, c_pad, dtype=dt, device=DEV)
+            lk.latent_attention(q, pg.cache, out, pos, pg.dev(range(len(lens) + 1)), pg.dev(pg.table), pg.dev(pg.cu), block_size=block,
+                                window=window, scale=0.2, max_kv_len=max(lens), n_splits=splits)
+            _close(out, want, dt, b16=1.5e-2)
+
+
 # ---- prompt portions ---------------------------------------------------------------------------
-@pytest.mark.parametrize("q_dim,r_pad,v_pad", [(32, 32, 32), (64, 32, 64), (64, 64, 128), (128, 32, 64), (128, 64, 128), (192, 64, 64)])
+@pytest.mark.parametrize("q_dim,r_pad,v_pad", [(32, 32, 32), (32, 64, 64), (64, 64, 128), (128, 32, 64), (128, 64, 128), (192, 64, 64)])
 @pytest.mark.parametrize("window", [0, 1, 40, 64, 129, 300])
 def test_portion_attention(q_dim, r_pad, v_pad, window):
     """Portions at several offsets of unequal sequences, with the context gathered and cut to the window by the plan."""

@@ -151,14 +151,16 @@ def main(argv=None):
             most = max([sum(q) for _, q, _ in cases] + sizes)
             m = dagupel(size, L, need) if D else llama(size, L, need * (BLOCK // 16), most)
             base = dict(size=size, model=which, layers=L)
+            # (the Llama step has no window: it decodes over as many keys as the window leaves the other)
+            context = args.context if D else min(args.context, window)
             for bs in sizes:
-                tokens, positions, params, _ = make_decode_inputs(bs, args.context, block, DEV, seed=1, vocab=vocab)
+                tokens, positions, params, _ = make_decode_inputs(bs, context, block, DEV, seed=1, vocab=vocab)
                 if D:
                     m.reserve_workspaces(bs)
                 else:
-                    m.reserve_workspaces(bs, args.context)
+                    m.reserve_workspaces(bs, context)
                 t = timed(lambda: m.forward(tokens, positions, params))
-                emit(kind="decode", **base, bs=bs, context=args.context, ms=t * 1e3, us_per_layer=t / L * 1e6, tokens_per_s=bs / t)
+                emit(kind="decode", **base, bs=bs, context=context, ms=t * 1e3, us_per_layer=t / L * 1e6, tokens_per_s=bs / t)
                 # the kernels of a layer
                 if D:
                     a0 = m.layers[0].attn
@@ -169,8 +171,8 @@ def main(argv=None):
                     def attn():
                         for c in m.caches:
                             lk.latent_attention(q, c.rows, o, positions, params.q_cu_seq_lens, params.block_tables, params.cu_block_lens,
-                                                block_size=BLOCK, window=window, scale=0.07, max_kv_len=args.context)
-                    seen = min(window, args.context)
+                                                block_size=BLOCK, window=window, scale=0.07, max_kv_len=context)
+                    seen = min(window, context)
                     nbytes, flops = bs * seen * R * 2, 2 * bs * seen * heads * (R + a0.c_pad)
                     h = torch.randn(bs, m.k_width, device=DEV).to(torch.bfloat16)
                     act = torch.randn(bs, ff, device=DEV).to(torch.bfloat16)
@@ -188,7 +190,7 @@ def main(argv=None):
                     def attn():
                         for x in m.layers:
                             m.attn.handler.batch_decode(q, x["kv"], params, -1, o)
-                    seen = args.context
+                    seen = context
                     nbytes, flops = bs * seen * kv_heads * 128 * 4, 4 * bs * seen * heads * 128
                     h = torch.randn(bs, width, device=DEV).to(torch.bfloat16)
                     act = torch.randn(bs, ff, device=DEV).to(torch.bfloat16)
