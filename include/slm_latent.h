@@ -1,7 +1,7 @@
 /*
  * slm_latent.h -- C ABI of libslm_latent.so: the MI355X (gfx950) kernels of the dense 16-/32-bit model
- * path with latent attention (scalellm_amd/dagupel.py is its model; the mechanisms are separate entry
- * points with their constants as arguments).
+ * path (residual stream, norms, products) and of latent attention (scalellm_amd/dagupel.py).  The mechanisms
+ * are separate entry points with their constants as arguments.
  *
  * Conventions are those of slm_hip.h: plain pointers and sizes, asynchronous on `stream`, nothing is
  * allocated or synchronised (hipGraph-capturable), 0 or a negative slm_status comes back.
@@ -24,7 +24,8 @@ SLM_API const char* slm_latent_version(void);
 SLM_API const char* slm_latent_status_string(int status);
 SLM_API const char* slm_latent_last_hip_error(void);
 
-/* ---- 1. fp32 residual stream: (embedding | add) + RMS norm --------------------------------------- */
+/* ---- 1. fp32 residual stream: (embedding | add) + norm -------------------------------------------- */
+/* norms: RMS x / sqrt(mean x^2 + eps) * weight;  TANH tanh(alpha x) * weight + bias                    */
 typedef struct slm_residual_norm_args {
   float* resid;             /* [rows, width] fp32, read and written (written only by EMBED)             */
   const void* delta;        /* ADD: [rows, width] of dtype, row stride ld_delta                         */
@@ -35,11 +36,14 @@ typedef struct slm_residual_norm_args {
   const void* pos_table;    /* EMBED: [max_positions, width] of dtype, or NULL                          */
   const int32_t* row_index; /* NULL, or [rows]: output row r is made of stream row row_index[r] (PLAIN) */
   const float* weight;      /* [width] fp32; NULL: only the sum, no norm                                */
+  const float* bias;        /* TANH: [width] fp32                                                       */
   void* out;                /* [rows, ld_out] of dtype; columns width .. ld_out-1 are zeroed            */
   int64_t rows, width, ld_delta, ld_embed, ld_out, slab_stride;
-  float eps;
-  int32_t n_slabs, mode, dtype;
+  float eps, norm_alpha;
+  float delta_mult;         /* factor of what is added: the delta, or the embedding row                 */
+  int32_t n_slabs, mode, dtype, norm;
 } slm_residual_norm_args;
+enum { SLM_NORM_RMS = 0, SLM_NORM_TANH = 1 };
 enum { SLM_RN_EMBED = 0, SLM_RN_ADD = 1, SLM_RN_SLABS = 2, SLM_RN_PLAIN = 3 };
 SLM_API int slm_residual_norm(const slm_residual_norm_args* a, void* stream);
 
@@ -47,20 +51,21 @@ SLM_API int slm_residual_norm(const slm_residual_norm_args* a, void* stream);
 /* x [batch][M, K], w [batch][N, K] (K contiguous, K % 64 == 0, N % 16 == 0).  Epilogues:               */
 /*   STORE   y[m, n] of dtype;  F32  y[m, n] = alpha * acc as fp32;                                     */
 /*   SLABS   y = fp32 [n_splits][M][ldy] partial sums (the consumer adds them, slm_residual_norm);      */
-/*   GLU     w = [gate | up] (N = 2 * half): y[m, n] = clamped_glu(gate, up), width half;               */
+/*   GLU     w = [gate | up] (N = 2 * half): y[m, n] = glu(gate, up) as below, width half;              */
 /*   GATE    y = acc * sigmoid(gate[m * ld_gate + batch index]) (per-head output gate).                 */
 typedef struct slm_linear_args {
   const void* x; const void* w; void* y; const void* gate;
   int64_t M, N, K, ldx, ldw, ldy, ld_gate;
   int64_t x_batch, w_batch, y_batch;   /* element strides between batch items                           */
-  float alpha, limit, glu_alpha;
+  float alpha, limit, glu_alpha, glu_shift;
   int32_t batch, n_splits, epilogue, dtype;
 } slm_linear_args;
 enum { SLM_LIN_STORE = 0, SLM_LIN_F32 = 1, SLM_LIN_SLABS = 2, SLM_LIN_GLU = 3, SLM_LIN_GATE = 4 };
 SLM_API int slm_linear(const slm_linear_args* a, void* stream);
-/* y = g sigmoid(alpha g) (u + 1), g = min(gate, limit), u = clamp(up, +-limit); gu = [rows, 2 * half]   */
+/* y = g sigmoid(alpha g) (u + shift), g = min(gate, limit), u = clamp(up, +-limit) (limit may be        */
+/* infinite: with alpha 1 and shift 0 the plain SiLU GLU); gu = [rows, 2 * half]                         */
 SLM_API int slm_clamped_glu(void* y, const void* gu, int64_t rows, int64_t half, int64_t ld_gu, int64_t ld_y,
-                            float limit, float glu_alpha, int32_t dtype, void* stream);
+                            float limit, float glu_alpha, float glu_shift, int32_t dtype, void* stream);
 
 /* ---- 3. latent cache append: latent RMS norm, rotation of the shared key part and of the queries --- */
 typedef struct slm_latent_append_args {

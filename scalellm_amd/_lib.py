@@ -12,6 +12,7 @@ import os
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "csrc", "libslm_hip.so")
 LATENT_LIB_PATH = os.path.join(_HERE, "csrc", "libslm_latent.so")
+MIXERS_LIB_PATH = os.path.join(_HERE, "csrc", "libslm_mixers.so")
 
 SLM_F16, SLM_BF16, SLM_F32 = 0, 1, 2   # (SLM_F32: libslm_latent only)
 SLM_W4_GPTQ, SLM_W4_AWQ = 0, 1
@@ -214,11 +215,12 @@ def _fields(*groups):
 
 class ResidualNormArgs(C.Structure):
     """slm_residual_norm_args."""
-    _fields_ = _fields((C.c_void_p, "resid delta slabs tokens positions embed pos_table row_index weight out"),
+    _fields_ = _fields((C.c_void_p, "resid delta slabs tokens positions embed pos_table row_index weight bias out"),
                        (C.c_int64, "rows width ld_delta ld_embed ld_out slab_stride"),
-                       (C.c_float, "eps"), (C.c_int32, "n_slabs mode dtype"))
+                       (C.c_float, "eps norm_alpha delta_mult"), (C.c_int32, "n_slabs mode dtype norm"))
 
 
+NORM_RMS, NORM_TANH = range(2)
 RN_EMBED, RN_ADD, RN_SLABS, RN_PLAIN = range(4)
 
 
@@ -226,7 +228,7 @@ class LinearArgs(C.Structure):
     """slm_linear_args."""
     _fields_ = _fields((C.c_void_p, "x w y gate"),
                        (C.c_int64, "M N K ldx ldw ldy ld_gate x_batch w_batch y_batch"),
-                       (C.c_float, "alpha limit glu_alpha"), (C.c_int32, "batch n_splits epilogue dtype"))
+                       (C.c_float, "alpha limit glu_alpha glu_shift"), (C.c_int32, "batch n_splits epilogue dtype"))
 
 
 LIN_STORE, LIN_F32, LIN_SLABS, LIN_GLU, LIN_GATE = range(5)
@@ -275,7 +277,7 @@ def latent_lib() -> C.CDLL:
         ("slm_latent_last_hip_error", C.c_char_p, []),
         ("slm_residual_norm", C.c_int, [P(ResidualNormArgs), ptr]),
         ("slm_linear", C.c_int, [P(LinearArgs), ptr]),
-        ("slm_clamped_glu", C.c_int, [ptr, ptr, i64, i64, i64, i64, f32, f32, i32, ptr]),
+        ("slm_clamped_glu", C.c_int, [ptr, ptr, i64, i64, i64, i64, f32, f32, f32, i32, ptr]),
         ("slm_latent_append", C.c_int, [P(LatentAppendArgs), ptr]),
         ("slm_latent_attn_workspace_bytes", C.c_size_t, [P(LatentAttnArgs)]),
         ("slm_latent_attn", C.c_int, [P(LatentAttnArgs), ptr]),
@@ -296,3 +298,86 @@ def latent_check(rc: int, what: str) -> None:
         L = latent_lib()
         detail = f" [{L.slm_latent_last_hip_error().decode()}]" if rc == -4 else ""
         raise SlmError(f"{what} failed: {L.slm_latent_status_string(rc).decode()} ({rc}){detail}")
+
+
+# ---- libslm_mixers.so (include/slm_mixers.h) -------------------------------------------------------
+REC_DELTA, REC_LIGHTNING = range(2)
+WINDOW_Q_TILE = 128
+
+
+class RecurrentArgs(C.Structure):
+    """slm_recurrent_args."""
+    _fields_ = _fields((C.c_void_p, "proj low conv_w conv_ring state neg_a dt_bias decay norm_weight positions q_cu state_slots "
+                                    "pre_qk pre_g pre_v pre_beta o out"),
+                       (C.c_int64, "rows ld_proj ld_low ld_out off_q off_k off_v off_b off_gate"),
+                       (C.c_int32, "mode dtype batch n_single n_slots heads qk_heads dim vdim dim_pad v_pad taps"),
+                       (C.c_float, "q_scale eps unit_eps"))
+
+
+class GatedNormArgs(C.Structure):
+    """slm_gated_norm_args."""
+    _fields_ = _fields((C.c_void_p, "o gate weight out"), (C.c_int64, "rows ld_gate ld_out out_width"),
+                       (C.c_int32, "heads vdim v_pad per_head dtype"), (C.c_float, "eps scale"))
+
+
+class WindowAppendArgs(C.Structure):
+    """slm_window_append_args."""
+    _fields_ = _fields((C.c_void_p, "proj key_cache value_cache q_weight k_weight cos_sin positions slots"),
+                       (C.c_int64, "rows ld_proj off_q off_k off_v max_positions n_slots"),
+                       (C.c_int32, "heads kv_heads dim rot d_pad v_pad dtype"), (C.c_float, "eps"))
+
+
+class WindowAttnArgs(C.Structure):
+    """slm_window_attn_args."""
+    _fields_ = _fields((C.c_void_p, "q key_cache value_cache out sink positions q_cu block_table block_cu workspace"),
+                       (C.c_size_t, "workspace_bytes"), (C.c_int64, "rows ld_q ld_out"),
+                       (C.c_int32, "batch heads kv_heads d_pad v_pad block_size window keep_first max_kv_len n_splits"),
+                       (C.c_float, "scale softcap out_scale"), (C.c_int32, "dtype generic"))
+
+
+class WindowPrefillArgs(C.Structure):
+    """slm_window_prefill_args."""
+    _fields_ = _fields((C.c_void_p, "q key_cache value_cache out sink slots tiles"), (C.c_int64, "ld_q ld_out n_rows n_ctx"),
+                       (C.c_int32, "n_tiles heads kv_heads d_pad v_pad window keep_first"), (C.c_float, "scale softcap out_scale"))
+
+
+_mixers = None
+
+
+def mixers_lib() -> C.CDLL:
+    """Load libslm_mixers.so or raise -- never falls back."""
+    global _mixers
+    if _mixers is not None:
+        return _mixers
+    if not os.path.exists(MIXERS_LIB_PATH):
+        raise SlmError(f"{MIXERS_LIB_PATH} not found: build it with `python -m scalellm_amd.build --library mixers`")
+    import torch  # noqa: F401  (one HIP runtime per process: see lib())
+    L = C.CDLL(MIXERS_LIB_PATH)
+    i32, ptr, P = C.c_int32, C.c_void_p, C.POINTER
+    for name, restype, argtypes in [
+        ("slm_mixers_version", C.c_char_p, []),
+        ("slm_mixers_status_string", C.c_char_p, [C.c_int]),
+        ("slm_mixers_last_hip_error", C.c_char_p, []),
+        ("slm_recurrent_dim_pad", i32, [i32]),
+        ("slm_recurrent_step", C.c_int, [P(RecurrentArgs), ptr]),
+        ("slm_recurrent_prepare", C.c_int, [P(RecurrentArgs), ptr]),
+        ("slm_recurrent_scan", C.c_int, [P(RecurrentArgs), ptr]),
+        ("slm_gated_norm", C.c_int, [P(GatedNormArgs), ptr]),
+        ("slm_window_append", C.c_int, [P(WindowAppendArgs), ptr]),
+        ("slm_window_attn_workspace_bytes", C.c_size_t, [P(WindowAttnArgs)]),
+        ("slm_window_attn", C.c_int, [P(WindowAttnArgs), ptr]),
+        ("slm_window_prefill", C.c_int, [P(WindowPrefillArgs), ptr]),
+        ("slm_window_prefill_supported", i32, [i32, i32]),
+    ]:
+        fn = getattr(L, name)
+        fn.restype = restype
+        fn.argtypes = argtypes
+    _mixers = L
+    return L
+
+
+def mixers_check(rc: int, what: str) -> None:
+    if rc != 0:
+        L = mixers_lib()
+        detail = f" [{L.slm_mixers_last_hip_error().decode()}]" if rc == -4 else ""
+        raise SlmError(f"{what} failed: {L.slm_mixers_status_string(rc).decode()} ({rc}){detail}")

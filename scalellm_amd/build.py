@@ -6,6 +6,7 @@
 
   hip     csrc/*.hip         -> csrc/libslm_hip.so      int4 / 8-bit linears, paged MHA, all-reduce
   latent  csrc/latent/*.hip  -> csrc/libslm_latent.so   dense 16- / 32-bit path, latent attention
+  mixers  csrc/mixers/*.hip  -> csrc/libslm_mixers.so   windowed attention with a sink, recurrent layers
 
 The .so files are git-ignored.
 """
@@ -26,8 +27,10 @@ INCLUDE = os.path.join(ROOT, "include")
 OBJ_DIR = os.path.join(CSRC, "build")
 LIB = os.path.join(CSRC, "libslm_hip.so")
 LATENT_LIB = os.path.join(CSRC, "libslm_latent.so")
+MIXERS_LIB = os.path.join(CSRC, "libslm_mixers.so")
 # library -> (source folder, result)
-LIBRARIES = {"hip": (CSRC, LIB), "latent": (os.path.join(CSRC, "latent"), LATENT_LIB)}
+LIBRARIES = {"hip": (CSRC, LIB), "latent": (os.path.join(CSRC, "latent"), LATENT_LIB),
+             "mixers": (os.path.join(CSRC, "mixers"), MIXERS_LIB)}
 ARCH = "gfx950"
 
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
@@ -46,7 +49,7 @@ def _sources(folder: str):
 
 
 def _deps_mtime(folder: str):
-    hdrs = [h for d in {folder, CSRC, INCLUDE} for h in glob.glob(os.path.join(d, "*.h"))]
+    hdrs = [h for d in {folder, CSRC, INCLUDE, os.path.join(CSRC, "latent") if folder != CSRC else CSRC} for h in glob.glob(os.path.join(d, "*.h"))]
     return max(os.path.getmtime(h) for h in hdrs)
 
 

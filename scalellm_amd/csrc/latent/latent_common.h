@@ -74,10 +74,10 @@ __device__ __forceinline__ float block_max256(float v, float* tmp) {
 }
 
 __device__ __forceinline__ float sigmoid_f32(float x) { return 1.0f / (1.0f + __expf(-x)); }
-__device__ __forceinline__ float clamped_glu_f32(float g, float u, float limit, float alpha) {
+__device__ __forceinline__ float clamped_glu_f32(float g, float u, float limit, float alpha, float shift) {
   g = fminf(g, limit);
   u = fminf(fmaxf(u, -limit), limit);
-  return g * sigmoid_f32(alpha * g) * (u + 1.0f);
+  return g * sigmoid_f32(alpha * g) * (u + shift);
 }
 
 // sequence of a query row: the last s with q_cu[s] <= row (batch >= 1)

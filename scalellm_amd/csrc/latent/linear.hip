@@ -147,7 +147,7 @@ __global__ void __launch_bounds__(256) linear_kernel(const slm_linear_args a) {
         reinterpret_cast<float*>(a.y)[item * a.y_batch + mm * a.ldy + nn] = a.alpha * total(t * MT + v);
       } else if constexpr (EPI == SLM_LIN_GLU) {
         reinterpret_cast<E*>(a.y)[mm * a.ldy + nn] =
-            (E)clamped_glu_f32(total(2 * t * MT + v), total((2 * t + 1) * MT + v), a.limit, a.glu_alpha);
+            (E)clamped_glu_f32(total(2 * t * MT + v), total((2 * t + 1) * MT + v), a.limit, a.glu_alpha, a.glu_shift);
       } else if constexpr (EPI == SLM_LIN_GATE) {
         const float gl = to_f32(reinterpret_cast<const E*>(a.gate)[mm * a.ld_gate + item]);
         reinterpret_cast<E*>(a.y)[item * a.y_batch + mm * a.ldy + nn] = (E)(total(t * MT + v) * sigmoid_f32(gl));

@@ -1,5 +1,5 @@
-// residual_norm.hip -- the fp32 residual stream: what a sub-layer adds (or the embedding), and the RMS
-// norm in front of the next projection, in one launch.  One workgroup per row; the row stays in
+// residual_norm.hip -- the fp32 residual stream: what a sub-layer adds (or the embedding), and the norm (RMS, or
+// tanh(alpha x), which needs no statistics) in front of the next projection, in one launch.  One workgroup per row; the row stays in
 // registers between the sum of squares and the scaling.  Bound: HBM, trivial.
 #include "latent_common.h"
 
@@ -39,13 +39,15 @@ __global__ void __launch_bounds__(RN_THREADS) residual_norm_kernel(const slm_res
 #pragma unroll
           for (int j = 0; j < V; ++j) x[s][j] += t[j];
         }
+#pragma unroll
+        for (int j = 0; j < V; ++j) x[s][j] *= a.delta_mult;
       } else {
         load_f32<V>(r + i, x[s]);
         if constexpr (MODE == SLM_RN_ADD) {
           float t[V];
           load_f32<V>(e0 + i, t);
 #pragma unroll
-          for (int j = 0; j < V; ++j) x[s][j] += t[j];
+          for (int j = 0; j < V; ++j) x[s][j] = __builtin_fmaf(t[j], a.delta_mult, x[s][j]);
         }
         if constexpr (MODE == SLM_RN_SLABS) {
           // (all slab loads of a chunk in flight at once)
@@ -65,7 +67,7 @@ __global__ void __launch_bounds__(RN_THREADS) residual_norm_kernel(const slm_res
                 for (int j = 0; j < V; ++j) d[j] += t[k][j];
           }
 #pragma unroll
-          for (int j = 0; j < V; ++j) x[s][j] += d[j];
+          for (int j = 0; j < V; ++j) x[s][j] = __builtin_fmaf(d[j], a.delta_mult, x[s][j]);
         }
       }
       if constexpr (MODE != SLM_RN_PLAIN) store_f32<V>(r + i, x[s]);
@@ -74,7 +76,8 @@ __global__ void __launch_bounds__(RN_THREADS) residual_norm_kernel(const slm_res
     }
   }
   if (!a.weight) return;  // (uniform: only the sum was asked for)
-  const float rs = 1.0f / sqrtf(block_sum256(ss, red) / (float)width + a.eps);
+  const bool rms = a.norm == SLM_NORM_RMS;
+  const float rs = rms ? 1.0f / sqrtf(block_sum256(ss, red) / (float)width + a.eps) : 0.f;
   E* o = reinterpret_cast<E*>(a.out) + row * a.ld_out;
 #pragma unroll
   for (int s = 0; s < RN_STEPS; ++s) {
@@ -84,6 +87,12 @@ __global__ void __launch_bounds__(RN_THREADS) residual_norm_kernel(const slm_res
       load_f32<V>(a.weight + i, w);
 #pragma unroll
       for (int j = 0; j < V; ++j) y[j] = x[s][j] * rs * w[j];
+      if (!rms) {
+        float b[V];
+        load_f32<V>(a.bias + i, b);
+#pragma unroll
+        for (int j = 0; j < V; ++j) y[j] = __builtin_fmaf(tanhf(a.norm_alpha * x[s][j]), w[j], b[j]);
+      }
       store_f32<V>(o + i, y);
     }
   }
@@ -92,7 +101,8 @@ __global__ void __launch_bounds__(RN_THREADS) residual_norm_kernel(const slm_res
 
 template <typename E>
 __global__ void __launch_bounds__(256) clamped_glu_kernel(E* __restrict__ y, const E* __restrict__ gu, int64_t half4,
-                                                          int64_t n4, int64_t ld_gu, int64_t ld_y, float limit, float alpha) {
+                                                          int64_t n4, int64_t ld_gu, int64_t ld_y, float limit, float alpha,
+                                                          float shift) {
   const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
   if (i >= n4) return;
   const int64_t row = i / half4, c = (i % half4) * 4;
@@ -100,7 +110,7 @@ __global__ void __launch_bounds__(256) clamped_glu_kernel(E* __restrict__ y, con
   load_f32<4>(gu + row * ld_gu + c, g);
   load_f32<4>(gu + row * ld_gu + half4 * 4 + c, u);
 #pragma unroll
-  for (int j = 0; j < 4; ++j) o[j] = clamped_glu_f32(g[j], u[j], limit, alpha);
+  for (int j = 0; j < 4; ++j) o[j] = clamped_glu_f32(g[j], u[j], limit, alpha, shift);
   store_f32<4>(y + row * ld_y + c, o);
 }
 
@@ -108,7 +118,7 @@ template <typename E, int MODE>
 static int rn_launch(const slm_residual_norm_args& a, hipStream_t st) {
   const bool v4 = a.width % 4 == 0 && a.ld_delta % 4 == 0 && a.ld_embed % 4 == 0 && a.ld_out % 4 == 0 &&
                   a.slab_stride % 4 == 0 && aligned16(a.resid) && aligned16(a.delta) && aligned16(a.slabs) &&
-                  aligned16(a.embed) && aligned16(a.pos_table) && aligned16(a.weight) && aligned16(a.out);
+                  aligned16(a.embed) && aligned16(a.pos_table) && aligned16(a.weight) && aligned16(a.bias) && aligned16(a.out);
   if (a.width > (v4 ? 4 : 1) * RN_THREADS * RN_STEPS) return SLM_ERR_UNSUPPORTED;
   hip_clear_error();
   if (v4) residual_norm_kernel<E, MODE, 4><<<dim3((unsigned)a.rows), dim3(RN_THREADS), 0, st>>>(a);
@@ -153,13 +163,14 @@ extern "C" SLM_API int slm_residual_norm(const slm_residual_norm_args* a, void* 
   if (a->mode == SLM_RN_ADD && (!a->delta || a->ld_delta < a->width)) return SLM_ERR_INVALID_ARG;
   if (a->mode == SLM_RN_SLABS && (!a->slabs || a->n_slabs < 1 || a->ld_delta < a->width)) return SLM_ERR_INVALID_ARG;
   if (a->weight ? (!a->out || a->ld_out < a->width) : a->mode == SLM_RN_PLAIN) return SLM_ERR_INVALID_ARG;
+  if (a->norm < 0 || a->norm > SLM_NORM_TANH || (a->weight && a->norm == SLM_NORM_TANH && !a->bias)) return SLM_ERR_INVALID_ARG;
   if (a->dtype == SLM_BF16) return rn_mode<bf16>(*a, (hipStream_t)stream);
   if (a->dtype == SLM_F32) return rn_mode<float>(*a, (hipStream_t)stream);
   return SLM_ERR_UNSUPPORTED;
 }
 
 extern "C" SLM_API int slm_clamped_glu(void* y, const void* gu, int64_t rows, int64_t half, int64_t ld_gu, int64_t ld_y,
-                                       float limit, float glu_alpha, int32_t dtype, void* stream) {
+                                       float limit, float glu_alpha, float glu_shift, int32_t dtype, void* stream) {
   if (!y || !gu || rows < 0 || half <= 0 || half % 4 || ld_gu < 2 * half || ld_gu % 4 || ld_y < half || ld_y % 4)
     return SLM_ERR_INVALID_ARG;
   if (!aligned16(y) || !aligned16(gu)) return SLM_ERR_ALIGNMENT;
@@ -168,9 +179,9 @@ extern "C" SLM_API int slm_clamped_glu(void* y, const void* gu, int64_t rows, in
   const dim3 grid((unsigned)((n4 + 255) / 256));
   hip_clear_error();
   if (dtype == SLM_BF16)
-    clamped_glu_kernel<bf16><<<grid, dim3(256), 0, (hipStream_t)stream>>>((bf16*)y, (const bf16*)gu, half4, n4, ld_gu, ld_y, limit, glu_alpha);
+    clamped_glu_kernel<bf16><<<grid, dim3(256), 0, (hipStream_t)stream>>>((bf16*)y, (const bf16*)gu, half4, n4, ld_gu, ld_y, limit, glu_alpha, glu_shift);
   else if (dtype == SLM_F32)
-    clamped_glu_kernel<float><<<grid, dim3(256), 0, (hipStream_t)stream>>>((float*)y, (const float*)gu, half4, n4, ld_gu, ld_y, limit, glu_alpha);
+    clamped_glu_kernel<float><<<grid, dim3(256), 0, (hipStream_t)stream>>>((float*)y, (const float*)gu, half4, n4, ld_gu, ld_y, limit, glu_alpha, glu_shift);
   else return SLM_ERR_UNSUPPORTED;
   return hip_check_launch();
 }

@@ -85,6 +85,8 @@ class _LayerWeights:
 
 @register_model("Dagupel")
 class DagupelStep:
+    libraries = ("latent",)
+
     def __init__(self, config: DagupelConfig, ckpt: Checkpoint, limits: ModelLimits):
         c = self.config = config
         if limits.dtype not in (torch.bfloat16, torch.float32):

@@ -1,14 +1,15 @@
 """The serving engine around a step model: paged block allocation, step building, continuous batching with chunked
 prompts, and generation.
 
-  BlockAllocator   free list of cache blocks (block tables hold first-slot ids: block * block_size)
-  Sequence         token ids, how many of them the cache holds, its blocks
+  BlockAllocator   free lists of cache blocks (block tables hold first-slot ids: block * block_size) and of the state
+                   slots of recurrent layers
+  Sequence         token ids, how many of them the cache holds, its blocks and its state slot
   StepBuilder      entries (sequence, new tokens) -> tokens, positions, InputParameters of ONE batch
   Scheduler        which sequences bring how many tokens into the next step
   LLMEngine        the loop: schedule -> ModelRunner.forward -> sample -> finish
 
 A step model is anything with forward(tokens, positions, params, return_logits=True) -> logits: DagupelStep,
-LlamaDecodeStep.
+VebusunStep, LlamaDecodeStep.
 """
 from __future__ import annotations
 
@@ -25,15 +26,18 @@ from .sampling import Sampler, SamplingParams
 
 
 class OutOfBlocks(RuntimeError):
-    """The cache pool has no free block left."""
+    """The cache pool has no free block (or state slot) left."""
 
 
 class BlockAllocator:
-    def __init__(self, n_blocks: int, block_size: int):
+    """n_states: recurrent state slots, one per live sequence (0: the model keeps none)."""
+
+    def __init__(self, n_blocks: int, block_size: int, n_states: int = 0):
         if block_size < 1 or block_size & (block_size - 1):
             raise ValueError("block_size is a power of two")
-        self.n_blocks, self.block_size = n_blocks, block_size
+        self.n_blocks, self.block_size, self.n_states = n_blocks, block_size, n_states
         self._free: Deque[int] = deque(range(n_blocks))
+        self._free_states: Deque[int] = deque(range(n_states))
 
     @property
     def n_free(self) -> int:
@@ -50,6 +54,22 @@ class BlockAllocator:
     def free(self, blocks: Seq[int]) -> None:
         self._free.extend(blocks)
 
+    @property
+    def n_free_states(self) -> int:
+        return len(self._free_states)
+
+    def can_admit(self, n_tokens: int) -> bool:
+        """Room for a new sequence of n_tokens tokens?"""
+        return self.blocks_for(n_tokens) <= self.n_free and (not self.n_states or bool(self._free_states))
+
+    def allocate_state(self) -> int:
+        if not self._free_states:
+            raise OutOfBlocks(f"all {self.n_states} state slots are taken")
+        return self._free_states.popleft()
+
+    def free_state(self, slot: int) -> None:
+        self._free_states.append(slot)
+
 
 @dataclass
 class Sequence:
@@ -57,18 +77,23 @@ class Sequence:
     tokens: List[int]
     n_cached: int = 0                 # tokens whose keys the cache holds
     blocks: List[int] = field(default_factory=list)
+    state: Optional[int] = None       # slot of its recurrent state
     n_prompt: int = 0
     sampler: Optional[Sampler] = None
 
     def reserve(self, allocator: BlockAllocator, n_tokens: int) -> None:
-        """Blocks for the first n_tokens tokens."""
+        """Blocks for the first n_tokens tokens, and a state slot where the model keeps state."""
         need = allocator.blocks_for(n_tokens) - len(self.blocks)
         if need > 0:
             self.blocks += allocator.allocate(need)
+        if allocator.n_states and self.state is None:
+            self.state = allocator.allocate_state()
 
     def release(self, allocator: BlockAllocator) -> None:
         allocator.free(self.blocks)
-        self.blocks, self.n_cached = [], 0
+        if self.state is not None:
+            allocator.free_state(self.state)
+        self.blocks, self.state, self.n_cached = [], None, 0
 
 
 @dataclass
@@ -121,6 +146,8 @@ class StepBuilder:
             kv_cu.append(kv_cu[-1] + c + n)
         arrays = [np.concatenate(tokens), np.concatenate(pos), np.concatenate(slots), np.concatenate(table),
                   np.asarray(bcu), np.asarray(q_cu), np.asarray(kv_cu)]
+        if self.allocator.n_states:
+            arrays.append(np.asarray([entries[i][0].state for i in order]))
         if logit_rows is not None:
             arrays.append(np.asarray([row0[i] + p for i in range(len(entries)) for p in logit_rows.get(i, ())], dtype=np.int32))
         # one transfer; every array starts on a 16-byte boundary of it
@@ -132,10 +159,11 @@ class StepBuilder:
         dev = torch.from_numpy(packed).to(self.device)
         d = [dev[int(s):int(s) + n] for s, n in zip(at, sizes)]
         kv_lens = np.diff(kv_cu)
+        state_slots = d[7] if self.allocator.n_states else None
         params = InputParameters(q_cu_seq_lens=d[5], kv_cu_seq_lens=d[6], new_cache_slots=d[2], block_tables=d[3],
                                  cu_block_lens=d[4], q_max_seq_len=max(n_new), kv_max_seq_len=int(kv_lens.max()),
-                                 kv_total_len=int(kv_cu[-1]), logit_rows=d[7] if logit_rows is not None else None,
-                                 portions=portions)
+                                 kv_total_len=int(kv_cu[-1]), logit_rows=d[-1] if logit_rows is not None else None,
+                                 portions=portions, state_slots=state_slots)
         return Step(d[0], d[1], params, row0, order)
 
     @staticmethod
@@ -193,7 +221,7 @@ class Scheduler:
                 budget -= n
         while self.waiting and not preempted and budget > 0 and len(self.running) < self.max_seqs:
             seq = self.waiting[0]
-            if self.allocator.blocks_for(len(seq.tokens)) > self.allocator.n_free:
+            if not self.allocator.can_admit(len(seq.tokens)):
                 break   # (a lone request always fits: LLMEngine.add_request)
             n = min(len(seq.tokens), budget)
             seq.reserve(self.allocator, n)
@@ -215,7 +243,7 @@ class LLMEngine:
     def __init__(self, model, n_blocks: int, block_size: int, device="cuda", options: Optional[EngineOptions] = None):
         self.model, self.device = model, torch.device(device)
         self.options = o = options or EngineOptions()
-        self.allocator = BlockAllocator(n_blocks, block_size)
+        self.allocator = BlockAllocator(n_blocks, block_size, getattr(model, "n_states", 0))
         self.builder = StepBuilder(self.allocator, self.device, getattr(model, "portion_min", None))
         self.scheduler = Scheduler(self.allocator, o.max_seqs, o.max_step_tokens)
         self.runner = ModelRunner(model, self.device, ModelRunnerOptions(

@@ -30,8 +30,6 @@ def main(argv=None) -> int:
     args = ap.parse_args(argv)
     prompts = [[int(t) for t in p.split(",") if t.strip()] for p in args.prompt]
 
-    from . import build
-    build.ensure("latent")
     import torch
     from .engine import EngineOptions, LLMEngine
     from .registry import ModelLimits, load_model
@@ -40,7 +38,8 @@ def main(argv=None) -> int:
     longest = max(len(p) for p in prompts) + args.max_tokens
     blocks = args.cache_tokens // B if args.cache_tokens else sum((len(p) + args.max_tokens + B - 1) // B for p in prompts)
     graphs = [int(g) for g in args.graphs.split(",") if g]
-    model = load_model(args.model, ModelLimits(max(blocks, 1), B, getattr(torch, args.dtype), "cuda"))
+    model = load_model(args.model, ModelLimits(max(blocks, 1), B, getattr(torch, args.dtype), "cuda", n_states=args.max_seqs,
+                                                max_positions=longest))
     engine = LLMEngine(model, max(blocks, 1), B, "cuda", EngineOptions(
         max_seqs=args.max_seqs, max_step_tokens=args.step_tokens, graph_batch_sizes=graphs, graph_max_seq_len=longest))
     engine.capture_graphs()

@@ -16,8 +16,8 @@ from .kernels import reserve_workspace
 
 # rows up to which the weight-streaming kernel serves a bf16 product; above it the vendor GEMM does
 STREAM_MAX_ROWS = 32
-# clamped GLU: y = g * sigmoid(alpha * g) * (u + 1)
-GLU_ALPHA = 1.702
+# clamped GLU: y = g * sigmoid(alpha * g) * (u + shift)
+GLU_ALPHA, GLU_SHIFT = 1.702, 1.0
 
 
 def _code(t: torch.Tensor) -> int:
@@ -49,6 +49,14 @@ def _i32(t: torch.Tensor, n: int, what: str) -> None:
     _need(t.dtype == torch.int32 and t.is_contiguous() and t.numel() >= n, f"{what}: contiguous int32 [>= {n}]")
 
 
+class TanhNorm:
+    """tanh(alpha x) * weight + bias in place of a norm's statistics; given to residual_norm() as its weight."""
+    __slots__ = ("alpha", "weight", "bias")
+
+    def __init__(self, alpha: float, weight: torch.Tensor, bias: torch.Tensor):
+        self.alpha, self.weight, self.bias = float(alpha), weight, bias
+
+
 class Slabs:
     """fp32 split-K partial sums [n, rows, ld] that residual_norm() adds up."""
     __slots__ = ("t",)
@@ -57,17 +65,17 @@ class Slabs:
         self.t = t
 
 
-def residual_norm(resid: torch.Tensor, out: Optional[torch.Tensor], weight: Optional[torch.Tensor], eps: float,
-                  delta=None, embed=None, row_index: Optional[torch.Tensor] = None) -> None:
-    """resid (fp32 [rows, width]) += delta (a [rows, >= width] tensor or Slabs), or
-    resid = table[tokens] (+ pos[positions]) for embed = (tokens, table, positions, pos); then
-    out = rms_norm(resid) * weight, zero padded to out's width.  weight = None: the sum only.
+def residual_norm(resid: torch.Tensor, out: Optional[torch.Tensor], weight, eps: float,
+                  delta=None, embed=None, row_index: Optional[torch.Tensor] = None, mult: float = 1.0) -> None:
+    """resid (fp32 [rows, width]) += mult * delta (a [rows, >= width] tensor or Slabs), or
+    resid = mult * (table[tokens] (+ pos[positions])) for embed = (tokens, table, positions, pos); then
+    out = rms_norm(resid) * weight, or a TanhNorm given as weight, zero padded to out's width.  weight = None: the sum only.
     row_index: out row r is the norm of stream row row_index[r]; nothing is added."""
     a = _lib.ResidualNormArgs()
     rows, width = resid.shape
     _need(resid.dtype == torch.float32 and resid.is_contiguous(), "residual_norm: resid is contiguous fp32")
     ref = out if out is not None else (delta if isinstance(delta, torch.Tensor) else None)
-    a.resid, a.width, a.eps = _p(resid), width, float(eps)
+    a.resid, a.width, a.eps, a.delta_mult = _p(resid), width, float(eps), float(mult)
     if embed is not None:
         tokens, table, positions, pos = embed
         _i32(tokens, rows, "tokens")
@@ -95,6 +103,10 @@ def residual_norm(resid: torch.Tensor, out: Optional[torch.Tensor], weight: Opti
             _i32(row_index, rows, "row_index")
             a.row_index = _p(row_index)
     a.rows = rows
+    if isinstance(weight, TanhNorm):
+        t, weight = weight, weight.weight
+        _need(t.bias.dtype == torch.float32 and t.bias.numel() == width and t.bias.is_contiguous(), "norm bias: fp32 [width]")
+        a.norm, a.norm_alpha, a.bias = _lib.NORM_TANH, t.alpha, _p(t.bias)
     if weight is not None:
         _need(weight.dtype == torch.float32 and weight.numel() == width and weight.is_contiguous(), "norm weight: fp32 [width]")
         _need(out.size(0) == rows and out.stride(1) == 1 and out.size(1) >= width, "residual_norm: out [rows, >= width]")
@@ -168,7 +180,8 @@ def linear_slabs(x: torch.Tensor, w: torch.Tensor) -> Slabs:
     return Slabs(out)
 
 
-def linear_glu(x: torch.Tensor, w_gate_up: torch.Tensor, out: torch.Tensor, limit: float, alpha: float = GLU_ALPHA) -> torch.Tensor:
+def linear_glu(x: torch.Tensor, w_gate_up: torch.Tensor, out: torch.Tensor, limit: float, alpha: float = GLU_ALPHA,
+               shift: float = GLU_SHIFT) -> torch.Tensor:
     """out = clamped GLU of the two halves of x [gate | up]^T: the activation is the product's epilogue where the
     streaming kernel runs, one more launch behind the vendor GEMM otherwise."""
     M, N, K = _check_xw(x, w_gate_up)
@@ -177,20 +190,21 @@ def linear_glu(x: torch.Tensor, w_gate_up: torch.Tensor, out: torch.Tensor, limi
     if streams_rows(x):
         a = _linear_args(x, w_gate_up, M, N, K)
         a.ldx, a.ldw, a.ldy, a.y, a.epilogue = x.stride(0), K, out.stride(0), _p(out), _lib.LIN_GLU
-        a.limit, a.glu_alpha = float(limit), float(alpha)
+        a.limit, a.glu_alpha, a.glu_shift = float(limit), float(alpha), float(shift)
         _run_linear(a)
     else:
         gu = torch.mm(x, w_gate_up.t())
-        clamped_glu(gu, out, limit, alpha)
+        clamped_glu(gu, out, limit, alpha, shift)
     return out
 
 
-def clamped_glu(gate_up: torch.Tensor, out: torch.Tensor, limit: float, alpha: float = GLU_ALPHA) -> None:
+def clamped_glu(gate_up: torch.Tensor, out: torch.Tensor, limit: float, alpha: float = GLU_ALPHA,
+                shift: float = GLU_SHIFT) -> None:
     M, N = gate_up.shape
     _need(out.shape == (M, N // 2) and gate_up.stride(1) == 1 and out.stride(1) == 1 and gate_up.dtype == out.dtype,
           "clamped_glu: gate_up [M, 2 n], out [M, n]")
     latent_check(_lib.latent_lib().slm_clamped_glu(_p(out), _p(gate_up), M, N // 2, gate_up.stride(0), out.stride(0), float(limit),
-                                                   float(alpha), _code(out), _stream()), "slm_clamped_glu")
+                                                   float(alpha), float(shift), _code(out), _stream()), "slm_clamped_glu")
 
 
 def linear_heads(x: torch.Tensor, x_head: int, w: torch.Tensor, out: torch.Tensor, out_head: int,

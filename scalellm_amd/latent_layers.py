@@ -232,10 +232,12 @@ class LatentAttention:
 # feed-forward
 # ---------------------------------------------------------------------------------------
 class ClampedGLU:
-    """W_down (g sigmoid(1.702 g) (u + 1)), g = min(W_gate h, limit), u = clamp(W_up h, +-limit)."""
+    """W_down (g sigmoid(alpha g) (u + shift)), g = min(W_gate h, limit), u = clamp(W_up h, +-limit); without a limit, with
+    alpha 1 and shift 0, the SiLU GLU."""
 
-    def __init__(self, width: int, ff: int, limit: float, w: Dict[str, torch.Tensor], dtype: torch.dtype, device):
-        self.limit = float(limit)
+    def __init__(self, width: int, ff: int, limit: float, w: Dict[str, torch.Tensor], dtype: torch.dtype, device,
+                 alpha: float = lk.GLU_ALPHA, shift: float = lk.GLU_SHIFT):
+        self.limit, self.alpha, self.shift = float(limit), float(alpha), float(shift)
         k, f = round_up(width, 64), round_up(ff, 64)
         self.w_gate_up = torch.zeros(2 * f, k, dtype=dtype, device=device)
         self.w_gate_up[:ff, :width] = w["gate"].to(device=device, dtype=dtype)
@@ -245,7 +247,7 @@ class ClampedGLU:
 
     def forward(self, h: torch.Tensor):
         act = h.new_empty(h.size(0), self.w_down.size(1))
-        lk.linear_glu(h, self.w_gate_up, act, self.limit)
+        lk.linear_glu(h, self.w_gate_up, act, self.limit, self.alpha, self.shift)
         if h.size(0) <= lk.STREAM_MAX_ROWS:
             return lk.linear_slabs(act, self.w_down)
         return lk.linear(act, self.w_down)

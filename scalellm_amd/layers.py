@@ -61,6 +61,8 @@ class InputParameters:
     # own for them (the rows in front of the first portion are single tokens).  Empty = nothing known: every row
     # is served on its own
     portions: Sequence[Portion] = ()
+    # extension: [batch] int32, the recurrent state every sequence owns (models with recurrent layers)
+    state_slots: Optional[torch.Tensor] = None
     # what a model derived from `portions` for this step (one entry per attention window)
     plans: Dict[object, object] = field(default_factory=dict)
 
@@ -85,14 +87,16 @@ def uniform_kv_hint(kv_total_len: int, n_seqs: int, q_max_seq_len: int, kv_max_s
 
 
 class KVCache:
-    """[n_blocks * block_size, n_kv_heads, head_dim] K and V tensors (memory/kv_cache.cpp:15-27)."""
+    """[n_blocks * block_size, n_kv_heads, head_dim] K and V tensors (memory/kv_cache.cpp:15-27); values may
+    have a width of their own."""
 
     def __init__(self, n_blocks: int, block_size: int, n_kv_heads: int, head_dim: int,
-                 dtype: torch.dtype, device):
+                 dtype: torch.dtype, device, value_dim: Optional[int] = None):
         self._block_size = block_size
         self.key_cache = torch.empty(n_blocks * block_size, n_kv_heads, head_dim, dtype=dtype,
                                      device=device)
-        self.value_cache = torch.empty_like(self.key_cache)
+        self.value_cache = torch.empty(n_blocks * block_size, n_kv_heads, value_dim or head_dim, dtype=dtype,
+                                       device=device)
 
     def block_size(self) -> int:
         return self._block_size
@@ -102,6 +106,17 @@ class KVCache:
 
     def set_kv_cache(self, slot_ids: torch.Tensor, keys: torch.Tensor, values: torch.Tensor) -> None:
         kernels.set_kv_cache(slot_ids, keys, values, self.key_cache, self.value_cache)
+
+
+class RecurrentState:
+    """What a recurrent layer keeps per sequence, one slot each (InputParameters.state_slots): an fp32 matrix per head
+    and, for layers with a short convolution, a ring of its last inputs (position p at p % taps).  A slot needs no
+    clearing: a row at position 0 starts from zero."""
+
+    def __init__(self, n_slots: int, heads: int, dim: int, vdim: int, device, taps: int = 0, channels: int = 0,
+                 dtype: torch.dtype = torch.float32):
+        self.state = torch.zeros(n_slots, heads, dim, vdim, dtype=torch.float32, device=device)
+        self.ring = torch.zeros(n_slots, taps, channels, dtype=dtype, device=device) if taps else None
 
 
 class HipAttnHandler:

@@ -63,7 +63,8 @@ class _Graph:
             q_cu_seq_lens=r.q_cu_seq_lens[:b + 1], kv_cu_seq_lens=r.kv_cu_seq_lens[:b + 1],
             new_cache_slots=r.new_cache_slots[:n], block_tables=r.block_tables,
             cu_block_lens=r.cu_block_lens[:b + 1], q_max_seq_len=r.options.num_decoding_tokens,
-            kv_max_seq_len=r.options.cuda_graph_max_seq_len)
+            kv_max_seq_len=r.options.cuda_graph_max_seq_len,
+            state_slots=None if r.state_slots is None else r.state_slots[:b])
         self.runner = runner
         # variant -> (graph, output); the key None is the reference's single graph
         self.variants: Dict[object, tuple] = {}
@@ -124,6 +125,8 @@ class _Graph:
         self.params.new_cache_slots.copy_(params.new_cache_slots, non_blocking=True)
         self.params.block_tables[:params.block_tables.numel()].copy_(params.block_tables, non_blocking=True)
         self.params.cu_block_lens.copy_(params.cu_block_lens, non_blocking=True)
+        if self.params.state_slots is not None:
+            self.params.state_slots.copy_(params.state_slots, non_blocking=True)
         key = None
         if None not in self.variants:   # the batch's own hints pick the variant (never the capture bound)
             key = self.runner.model.graph_variant_for(self.n_tokens, params)
@@ -174,6 +177,9 @@ class ModelRunner:
             per_seq = (options.cuda_graph_max_seq_len + options.block_size - 1) // options.block_size + 1
             self.block_tables = torch.zeros(mb * per_seq, **i32)
             self.cu_block_lens = torch.zeros(mb + 1, **i32)
+            # extension: models with recurrent layers (the capture runs write to these slots: capture before serving)
+            n_states = getattr(model, "n_states", 0)
+            self.state_slots = torch.arange(mb, **i32) % n_states if n_states else None
 
     def _run(self, tokens, positions, params):
         return self.model.forward(tokens, positions, params, **self.forward_kwargs)

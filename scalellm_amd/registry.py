@@ -4,7 +4,9 @@ A registered class has
     from_checkpoint(config: dict, checkpoint: Checkpoint, limits: ModelLimits) -> step model
 and a step model has
     forward(tokens, positions, params: InputParameters, return_logits: bool) -> next ids | logits
-    max_positions, vocab, and optionally portion_min (see engine.StepBuilder).
+    max_positions, vocab, and optionally portion_min (see engine.StepBuilder) and n_states (recurrent state slots: one per
+    live sequence, see engine.BlockAllocator).
+The class names the kernel libraries it runs on (`libraries`); load_model() compiles those that are not built yet.
 """
 from __future__ import annotations
 
@@ -15,10 +17,11 @@ from typing import Dict
 
 import torch
 
+from . import build
 from .checkpoint import Checkpoint, load_config
 
 # modules that register models when imported
-_MODULES = ("dagupel",)
+_MODULES = ("dagupel", "vebusun")
 _MODELS: Dict[str, type] = {}
 
 
@@ -29,6 +32,8 @@ class ModelLimits:
     block_size: int
     dtype: torch.dtype = torch.bfloat16
     device: str = "cuda"
+    n_states: int = 64       # live sequences a recurrent model keeps state for
+    max_positions: int = 0   # longest sequence of a model without a limit of its own; 0 = what the pool holds
 
 
 def register_model(name: str):
@@ -58,4 +63,6 @@ def architecture_of(config: dict) -> str:
 def load_model(path: str, limits: ModelLimits):
     config = load_config(path)
     cls = model_class(architecture_of(config))
+    for library in cls.libraries:
+        build.ensure(library)
     return cls.from_checkpoint(config, Checkpoint.open(os.path.join(path, "model.safetensors")), limits)

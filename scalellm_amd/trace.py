@@ -6,7 +6,7 @@ Steps come as JSON lines on standard input:
     {"step": 0, "entries": [{"id": "a", "tokens": [5, 17, 3], "want": [0, 2]}], "end": []}
 All entries of a step are one batch of LLMEngine.run_entries.  Wanted logits go to OUT/<step>.f32 (little-endian
 fp32 [wanted, vocab], entries and places in the given order); "done <step>" is printed after every step.  Requests
-named in "end" give their cache blocks back.  --max-tokens sizes the pool: the most tokens live requests hold, each
+named in "end" give their cache blocks and state back.  --max-tokens sizes the pool: the most tokens live requests hold, each
 rounded up to the block size.
 """
 from __future__ import annotations
@@ -28,8 +28,6 @@ def main(argv=None) -> int:
     ap.add_argument("--max-tokens", required=True, type=int, help="size of the cache pool in tokens")
     args = ap.parse_args(argv)
 
-    from . import build
-    build.ensure("latent")
     import torch
     from .engine import EngineOptions, LLMEngine, Sequence
     from .registry import ModelLimits, load_model
@@ -37,7 +35,7 @@ def main(argv=None) -> int:
         print("trace_run needs a GPU", file=sys.stderr)
         return 2
     n_blocks = max(1, (args.max_tokens + BLOCK_SIZE - 1) // BLOCK_SIZE)
-    limits = ModelLimits(n_blocks, BLOCK_SIZE, getattr(torch, args.dtype), "cuda")
+    limits = ModelLimits(n_blocks, BLOCK_SIZE, getattr(torch, args.dtype), "cuda", n_states=MAX_REQUESTS)
     engine = LLMEngine(load_model(args.model, limits), n_blocks, BLOCK_SIZE, "cuda", EngineOptions(max_seqs=MAX_REQUESTS))
     live = {}
     for line in sys.stdin:

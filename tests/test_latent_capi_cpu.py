@@ -65,7 +65,7 @@ def test_invalid_arguments_come_back_as_status():
     b.block_size, b.dtype = 16, 0
     assert L.slm_latent_attn(C.byref(b), None) == -2
     assert L.slm_latent_gather(None, None, None, 1, 64, None) == -1
-    assert L.slm_clamped_glu(4096, 4096, 1, 6, 12, 8, 1.0, 1.0, _lib.SLM_BF16, None) == -1
+    assert L.slm_clamped_glu(4096, 4096, 1, 6, 12, 8, 1.0, 1.0, 1.0, _lib.SLM_BF16, None) == -1
     p = _lib.LatentPrefillArgs()
     assert L.slm_latent_prefill(C.byref(p), None) == -1
     assert L.slm_latent_prefill_supported(128, 64, 128) == 1 and L.slm_latent_prefill_supported(250, 96, 128) == 0
