@@ -491,18 +491,23 @@ def main():
         # the latent-attention design beside the Llama step at equal size: lines of its own
         from tools.bench_dagupel import main as bench_dagupel
         raise SystemExit(bench_dagupel(rest))
+    if known.model == "vebusun":
+        # the delta-rule / parallel-mixer design beside the Dagupel and Llama steps at equal size: lines of its own
+        from tools.bench_vebusun import main as bench_vebusun
+        raise SystemExit(bench_vebusun(rest))
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=10)
     ap.add_argument("--warmup", type=int, default=3)
     ap.add_argument("--bits", type=int, default=4, choices=[4, 8], help="weight bits of the quantised linears "
                     "(8 = the reference's num_bits = 8 path: two int4 planes on the int4 kernels; not the BASELINE metric)")
-    ap.add_argument("--model", default="8b", choices=["8b", "70b", "dagupel"], help="8b = Llama-3-8B-shaped, "
+    ap.add_argument("--model", default="8b", choices=["8b", "70b", "dagupel", "vebusun"], help="8b = Llama-3-8B-shaped, "
                     "AWQ int4 g128, bs=256 (BASELINE.json metric configuration, configs[1]/[2]); 70b = "
                     "Llama-3-70B-shaped (in-tree defaults models/meta/llama.h:348-362), GPTQ symmetric "
                     "int4 g128, bs=128, TP = --gpus (configs[3]; TP=1 fits one MI355X: 35 GB of weights "
                     "+ 172 GB of KV); dagupel = prefill / decode lines of the latent-attention design beside the Llama step "
-                    "(options of its own: tools/bench_dagupel.py)")
+                    "(options of its own: tools/bench_dagupel.py); vebusun = the same for the delta-rule / parallel-mixer "
+                    "design (tools/bench_vebusun.py)")
     ap.add_argument("--bs", type=int, default=0, help="default 256 (8b) / 128 (70b)")
     ap.add_argument("--seqlen", type=int, default=4096)
     ap.add_argument("--block", type=int, default=16)

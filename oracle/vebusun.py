@@ -60,7 +60,8 @@ def sink_attention(h, w, m, eps):
         for a in range(H):
             g = a // (H // G)
             s = k[js, g] @ q[i, a] * m["scale"]
-            s = m["softcap"] * np.tanh(s / m["softcap"])
+            if m.get("softcap"):
+                s = m["softcap"] * np.tanh(s / m["softcap"])
             top = max(s.max(), w["sink"][a])
             p = np.exp(s - top)
             out[i, a] = p @ v[js, g] / (p.sum() + np.exp(w["sink"][a] - top))

@@ -77,7 +77,7 @@ def write_model(path, cfg, tensors):
     names = {torch.bfloat16: "BF16", torch.float32: "F32", torch.int32: "I32"}
     header, blobs, at = {}, [], 0
     for k, v in tensors.items():
-        raw = v.contiguous().view(torch.uint8).numpy().tobytes() if v.numel() else b""
+        raw = v.contiguous().view(-1).view(torch.uint8).numpy().tobytes() if v.numel() else b""
         header[k] = {"dtype": names[v.dtype], "shape": list(v.shape), "data_offsets": [at, at + len(raw)]}
         blobs.append(raw)
         at += len(raw)

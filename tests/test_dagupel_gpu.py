@@ -39,12 +39,12 @@ def row_errors_at(got, want, start, n):
     return np.sqrt((d * d).mean(-1)) / np.sqrt((w * w).mean())
 
 
-def _engine(cfg, tensors, dtype, n_blocks=16, block_size=16, **options):
+def _engine(cfg, tensors, dtype, n_blocks=16, block_size=16, n_states=64, **options):
     from scalellm_amd.checkpoint import Checkpoint
     from scalellm_amd.engine import EngineOptions, LLMEngine
     from scalellm_amd.registry import ModelLimits, model_class
     cls = model_class(cfg["architecture"])
-    model = cls.from_checkpoint(cfg, Checkpoint(dict(tensors)), ModelLimits(n_blocks, block_size, dtype, "cuda"))
+    model = cls.from_checkpoint(cfg, Checkpoint(dict(tensors)), ModelLimits(n_blocks, block_size, dtype, "cuda", n_states))
     return LLMEngine(model, n_blocks, block_size, "cuda", EngineOptions(**options))
 
 

@@ -276,3 +276,67 @@ def test_sampling_parameters():
     assert [a.sample(x) for _ in range(20)] == [b.sample(x) for _ in range(20)]
     with pytest.raises(ValueError):
         SamplingParams(top_p=0.0)
+
+
+def test_state_slots_are_owned_by_live_sequences():
+    """One slot per sequence from its first step to its end; a step names them in batch order; admission waits for one."""
+    alloc = BlockAllocator(40, 4, n_states=2)
+    a, b, c = (Sequence(n, list(range(9))) for n in "abc")
+    step = StepBuilder(alloc, "cpu", portion_min=2).build([(a, 5), (b, 1)])
+    assert step.order == [1, 0] and step.params.state_slots.tolist() == [b.state, a.state] and {a.state, b.state} == {0, 1}
+    with pytest.raises(OutOfBlocks):
+        c.reserve(alloc, 1)
+    assert not alloc.can_admit(1)
+    held = a.state
+    c.release(alloc)
+    a.release(alloc)
+    assert a.state is None and alloc.n_free_states == 1
+    c.reserve(alloc, 1)
+    assert c.state == held
+    step = StepBuilder(alloc, "cpu", portion_min=2).build([(b, 2), (c, 3)], {0: [1], 1: [0, 2]})
+    assert step.params.state_slots.tolist() == [b.state, c.state] and step.params.logit_rows.tolist() == [1, 2, 4]
+    s = Scheduler(BlockAllocator(40, 4, n_states=2), 8, 64)
+    for n in range(3):
+        s.add(Sequence(n, [1, 2, 3]))
+    assert [e[0].id for e in s.schedule()] == [0, 1]
+    s.finish(s.running[0])
+    assert [e[0].id for e in s.schedule()][-1] == 2
+    assert StepBuilder(BlockAllocator(4, 4), "cpu").build([(Sequence("x", [1]), 1)]).params.state_slots is None
+
+
+@pytest.mark.parametrize("start,q,size,keep", [(0, 300, 70, 5), (0, 300, 70, 100), (130, 140, 64, 3), (130, 140, 0, 0), (500, 1, 16, 0), (40, 2, 64, 30)])
+def test_window_plan_covers_what_the_rows_see(start, q, size, keep):
+    from oracle import vebusun as ref
+    from scalellm_amd.layers import Portion
+    from scalellm_amd.mixer_layers import WindowPlan
+    B, rng = 16, np.random.default_rng(0)
+    ps, row = [], 0
+    for extra in (0, 7):
+        n = start + q + extra
+        ps.append(Portion(row, q + extra, n, rng.permutation(200)[:(n + B - 1) // B].astype(np.int32) * B))
+        row += q + extra
+    slots, tiles = WindowPlan.host(ps, size, keep, B)
+    seen = set()
+    for row0, rows, base, n, kept, first, pos0 in tiles.tolist():
+        p = next(p for p in ps if p.row0 <= row0 < p.row0 + p.q_len)
+        at = {(j if j < kept else j + first - kept): int(slots[base + j]) for j in range(n)}
+        for r in range(rows):
+            assert pos0 + r == p.kv_len - p.q_len + row0 - p.row0 + r
+            seen.add(row0 + r)
+            for j in ref.visible(pos0 + r, {"size": size, "keep_first": keep}):
+                assert at[j] == int(p.blocks[j // B]) + j % B
+    assert seen == set(range(row)) and max(t[1] for t in tiles.tolist()) <= 128
+
+
+def test_vebusun_configuration():
+    from scalellm_amd.vebusun import VebusunConfig
+    from .vebusun_common import CONFIGS
+    c = VebusunConfig.parse(CONFIGS["odd"])
+    assert c.runs == [0, 1, 2, 1, 2, 1, 2] and c.layers[1].ff is None and c.layers[1].mixer.left.window == 21
+    assert VebusunConfig.parse(CONFIGS["tiny"]).runs == [0, 1]
+    bad = dict(CONFIGS["tiny"], loop={"start": 1, "stop": 5, "times": 2})
+    with pytest.raises(ValueError):
+        VebusunConfig.parse(bad)
+    bad = dict(CONFIGS["tiny"], layers=[dict(CONFIGS["tiny"]["layers"][0], type="other")])
+    with pytest.raises(ValueError):
+        VebusunConfig.parse(bad)
