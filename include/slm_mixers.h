@@ -47,18 +47,18 @@ typedef struct slm_recurrent_args {
   const int32_t* positions;  /* [rows]                                                                      */
   const int32_t* q_cu;       /* [batch + 1]                                                                 */
   const int32_t* state_slots;/* [batch]                                                                     */
-  float* pre_qk;             /* prepare -> scan: [portion rows][qk_heads][2][dim_pad]                       */
-  float* pre_g;              /* DELTA: [portion rows][heads][dim_pad]                                       */
-  float* pre_v;              /* [portion rows][heads][v_pad]                                                */
-  float* pre_beta;           /* DELTA: [portion rows][heads]                                                */
+  const int32_t* chunks;     /* prepare: [n_chunks][3]: sequence, first row, rows (<= 16) of every portion's chunks */
+  const int32_t* seq_chunks; /* scan: [batch - n_single]: a portion's first chunk (its chunks follow each other) */
+  float* pre;                /* prepare -> scan: [n_chunks][heads] records of slm_recurrent_record_floats   */
   float* o;                  /* scan: [portion rows][heads][v_pad]; step, LIGHTNING: [n_single][heads][v_pad] */
   void* out;                 /* step, DELTA: [n_single, ld_out] of dtype, [heads][vdim], zero padded to ld_out */
   int64_t rows, ld_proj, ld_low, ld_out, off_q, off_k, off_v, off_b, off_gate;
-  int32_t mode, dtype, batch, n_single, n_slots, heads, qk_heads, dim, vdim, dim_pad, v_pad, taps;
+  int32_t mode, dtype, batch, n_single, n_slots, heads, qk_heads, dim, vdim, dim_pad, v_pad, taps, n_chunks;
   float q_scale, eps, unit_eps;
 } slm_recurrent_args;
 /* the padded key width of the state for `dim` (0: not served), v_pad = vdim rounded up to 16 (at most 256) */
 SLM_API int32_t slm_recurrent_dim_pad(int32_t dim);
+SLM_API int64_t slm_recurrent_record_floats(int32_t dim_pad, int32_t v_pad);
 SLM_API int slm_recurrent_step(const slm_recurrent_args* a, void* stream);
 SLM_API int slm_recurrent_prepare(const slm_recurrent_args* a, void* stream);
 SLM_API int slm_recurrent_scan(const slm_recurrent_args* a, void* stream);

@@ -308,9 +308,9 @@ WINDOW_Q_TILE = 128
 class RecurrentArgs(C.Structure):
     """slm_recurrent_args."""
     _fields_ = _fields((C.c_void_p, "proj low conv_w conv_ring state neg_a dt_bias decay norm_weight positions q_cu state_slots "
-                                    "pre_qk pre_g pre_v pre_beta o out"),
+                                    "chunks seq_chunks pre o out"),
                        (C.c_int64, "rows ld_proj ld_low ld_out off_q off_k off_v off_b off_gate"),
-                       (C.c_int32, "mode dtype batch n_single n_slots heads qk_heads dim vdim dim_pad v_pad taps"),
+                       (C.c_int32, "mode dtype batch n_single n_slots heads qk_heads dim vdim dim_pad v_pad taps n_chunks"),
                        (C.c_float, "q_scale eps unit_eps"))
 
 
@@ -359,6 +359,7 @@ def mixers_lib() -> C.CDLL:
         ("slm_mixers_status_string", C.c_char_p, [C.c_int]),
         ("slm_mixers_last_hip_error", C.c_char_p, []),
         ("slm_recurrent_dim_pad", i32, [i32]),
+        ("slm_recurrent_record_floats", C.c_int64, [i32, i32]),
         ("slm_recurrent_step", C.c_int, [P(RecurrentArgs), ptr]),
         ("slm_recurrent_prepare", C.c_int, [P(RecurrentArgs), ptr]),
         ("slm_recurrent_scan", C.c_int, [P(RecurrentArgs), ptr]),

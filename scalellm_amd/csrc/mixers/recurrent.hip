@@ -3,11 +3,10 @@
 //
 //   step     one row per sequence: convolution, activations, unit vectors, gates, the update and (delta) the output norm
 //            in one launch.  One workgroup per (row, head); the state is read and written once.  Bound: HBM (state).
-//   prepare  rows of portions: the same inputs, activated and normed, to fp32 buffers.  Bound: HBM.
-//   scan     portions: the recurrence, token after token.  The columns of S are independent given q, k, g, so a wave
-//            owns 4 CPL of them: lane = (column, row group of 16), the state stays in registers from the portion's first
-//            token to its last, both contractions over key channels are register sums and one 16-lane DPP reduction,
-//            and no wave waits for another but at the chunks of inputs staged in LDS.  Bound: VALU.
+//   prepare  portions, cut into chunks of 16 tokens, every chunk at once: inputs activated and normed, decays summed, and
+//            what a chunk's tokens do to each other solved (a 16 x 16 triangular system).  Bound: VALU, HBM.
+//   scan     portions: chunk after chunk.  The columns of S are independent, so a workgroup owns 16 of them and keeps them
+//            in registers from the portion's first token to its last; the products are 32-bit MFMAs.  Bound: fp32 MFMA.
 //   gated_norm  the norm and gate behind a scan.
 #include "latent/latent_common.h"
 #include "slm_mixers.h"
@@ -43,9 +42,9 @@ __device__ __forceinline__ E raw_input(const slm_recurrent_args& a, int64_t row,
   return reinterpret_cast<const E*>(a.proj)[row * a.ld_proj + col];
 }
 template <typename E>
-__device__ __forceinline__ float decay_gate(const slm_recurrent_args& a, int64_t row, int head, int c) {
+__device__ __forceinline__ float decay_exponent(const slm_recurrent_args& a, int64_t row, int head, int c) {
   const float x = to_f32(reinterpret_cast<const E*>(a.low)[row * a.ld_low + (int64_t)head * a.dim + c]);
-  return expf(a.neg_a[head] * softplus_f32(x + a.dt_bias[head * a.dim + c]));
+  return a.neg_a[head] * softplus_f32(x + a.dt_bias[head * a.dim + c]);
 }
 
 // ---------------------------------------------------------------------------------------
@@ -86,7 +85,7 @@ __global__ void __launch_bounds__(1024) recurrent_step_kernel(const slm_recurren
         const int c = qh * a.dim + i;
         q = conv_input<E>(a, ring, row, row, p, c);
         k = conv_input<E>(a, ring, row, row, p, qk + c);
-        g = decay_gate<E>(a, row, head, i);
+        g = expf(decay_exponent<E>(a, row, head, i));
         if (first_of_group) {
           keep[c] = raw_input<E>(a, row, c);
           keep[qk + c] = raw_input<E>(a, row, qk + c);
@@ -218,216 +217,257 @@ __global__ void __launch_bounds__(1024) recurrent_step_kernel(const slm_recurren
 }
 
 // ---------------------------------------------------------------------------------------
-// prepare: one wave per (portion row, vector): q and k of every q/k head, v of every head, decays of every head
+// portions: chunks of 16 tokens
 // ---------------------------------------------------------------------------------------
-template <typename E, int MODE>
+// With L_t the sum of a chunk's log decays up to token t, S0 the state in front of it, x.d = product per key channel:
+//   (I + diag(beta) A) U = diag(beta) (V - Kd S0)     A_ts = sum_d k_t k_s exp(L_t - L_s), s < t;  Kd_t = k_t exp(L_t)
+//   O  = Qd S0 + B U                                  B_ts = sum_d q_t k_s exp(L_t - L_s), s <= t; Qd_t = q_t exp(L_t)
+//   S1 = diag(exp(L_end)) S0 + Kr^T U                 Kr_t = k_t exp(L_end - L_t)
+// Every exponent is <= 0: nothing overflows however fast a channel forgets.  Without the delta rule U = V.
+// A chunk's record for one head, in floats:
+//   Kd [16][DK] | Qd [16][DK] | Kr^T [DK][16] | exp(L_end) [DK] | V [16][v_pad] | T = (I + diag(beta) A)^-1 diag(beta) [16][16]
+//   | B [16][16]
+template <int DK>
+struct ChunkRecord {
+  static constexpr int KD = 0, QD = 16 * DK, KR = 32 * DK, GE = 48 * DK, V = 49 * DK;
+  int v_pad;
+  __device__ __forceinline__ int t() const { return V + 16 * v_pad; }
+  __device__ __forceinline__ int b() const { return t() + 256; }
+  __device__ __forceinline__ int64_t size() const { return b() + 256; }
+};
+
+// one workgroup per (chunk, head); every chunk of the step at once
+template <typename E, int MODE, int DK>
 __global__ void __launch_bounds__(256) recurrent_prepare_kernel(const slm_recurrent_args a) {
-  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-  const int64_t pr = blockIdx.x, row = pr + a.n_single;
-  const int s = seq_of_row(a.q_cu, a.batch, (int)row);
-  const int64_t row0 = a.q_cu[s];
-  const int p = a.positions[row];
-  const int n_tasks = 2 * a.qk_heads + (DELTA_MODE(MODE) ? 2 : 1) * a.heads;
-  const int qk = a.qk_heads * a.dim;
-  const E* ring = nullptr;
-  if constexpr (DELTA_MODE(MODE))
-    ring = reinterpret_cast<const E*>(a.conv_ring) + (int64_t)a.state_slots[s] * a.taps * (2 * (int64_t)qk + (int64_t)a.heads * a.vdim);
-  const E* in = reinterpret_cast<const E*>(a.proj) + row * a.ld_proj;
-  for (int task = blockIdx.y * 4 + wave; task < n_tasks; task += 4 * gridDim.y) {
-    if (task < 2 * a.qk_heads) {
-      const int h = task >> 1, which = task & 1;
-      float x[4], ss = 0.f;
-#pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const int c = lane + 64 * j;
-        x[j] = 0.f;
-        if (c < a.dim) {
-          if constexpr (DELTA_MODE(MODE)) x[j] = conv_input<E>(a, ring, row, row0, p, which * qk + h * a.dim + c);
-          else x[j] = silu_f32(to_f32(in[(which ? a.off_k : a.off_q) + h * a.dim + c]));
-        }
-        ss = __builtin_fmaf(x[j], x[j], ss);
-      }
-      float f = 1.0f;
-      if constexpr (DELTA_MODE(MODE)) f = (which ? 1.0f : a.q_scale) / sqrtf(wave_sum(ss) + a.unit_eps);
-      float* dst = a.pre_qk + ((pr * a.qk_heads + h) * 2 + which) * a.dim_pad;
-#pragma unroll
-      for (int j = 0; j < 4; ++j)
-        if (lane + 64 * j < a.dim_pad) dst[lane + 64 * j] = x[j] * f;
-    } else if (task < 2 * a.qk_heads + a.heads) {
-      const int h = task - 2 * a.qk_heads;
-      float* dst = a.pre_v + (pr * a.heads + h) * a.v_pad;
-      for (int c = lane; c < a.v_pad; c += 64) {
-        float v = 0.f;
-        if (c < a.vdim) {
-          if constexpr (DELTA_MODE(MODE)) v = conv_input<E>(a, ring, row, row0, p, 2 * qk + h * a.vdim + c);
-          else v = silu_f32(to_f32(in[a.off_v + h * a.vdim + c]));
-        }
-        dst[c] = v;
-      }
-      if constexpr (DELTA_MODE(MODE))
-        if (lane == 0) a.pre_beta[pr * a.heads + h] = sigmoid_full(to_f32(in[a.off_b + h]));
-    } else if constexpr (DELTA_MODE(MODE)) {
-      const int h = task - 2 * a.qk_heads - a.heads;
-      float* dst = a.pre_g + (pr * a.heads + h) * a.dim_pad;
-      for (int c = lane; c < a.dim_pad; c += 64) dst[c] = c < a.dim ? decay_gate<E>(a, row, h, c) : 1.0f;
-    }
-  }
-}
-
-// ---------------------------------------------------------------------------------------
-// scan: workgroup = (sequence, head, 16 CPL columns); DK = 16 R
-// ---------------------------------------------------------------------------------------
-template <int R>
-__device__ __forceinline__ void load_rows(const float* base, int rg, float (&x)[R]) {
-  if constexpr (R == 2) {
-    const f32x2 t = *reinterpret_cast<const f32x2*>(base + 2 * rg);
-    x[0] = t.x, x[1] = t.y;
-  } else {
-#pragma unroll
-    for (int i = 0; i < R / 4; ++i) {
-      const f32x4 t = *reinterpret_cast<const f32x4*>(base + 64 * i + 4 * rg);
-#pragma unroll
-      for (int j = 0; j < 4; ++j) x[4 * i + j] = t[j];
-    }
-  }
-}
-template <int R>
-__device__ __forceinline__ int row_of(int rg, int r) { return R == 2 ? 2 * rg + r : 64 * (r >> 2) + 4 * rg + (r & 3); }
-
-template <typename E, int MODE, int R, int CPL>
-__global__ void __launch_bounds__(256) recurrent_scan_kernel(const slm_recurrent_args a) {
   constexpr bool DELTA = DELTA_MODE(MODE);
-  constexpr int DK = 16 * R, NV = DELTA ? 3 : 2, COLS = 16 * CPL;
-  constexpr int TC = R > 8 ? 8 : 16;                   // tokens of a staged chunk
-  constexpr int ROWF = NV * DK + COLS;                 // floats a token brings: q | k | g | v
-  constexpr int V4 = TC * ROWF / 4, PER = (V4 + 255) / 256;
-  __shared__ __attribute__((aligned(16))) float buf[2][TC * ROWF];
-  __shared__ float sbeta[2][TC];
+  constexpr int LD = DK + 1;                     // (odd: the 16 rows a half-wave reads are in different banks)
+  __shared__ float sq[16 * LD], sk[16 * LD], sL[16 * LD], sa[16][17], sbeta[16];
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int n_cb = (a.v_pad + COLS - 1) / COLS;
-  const int cb = blockIdx.x % n_cb, head = blockIdx.x / n_cb % a.heads, seq = a.n_single + blockIdx.x / (n_cb * a.heads);
-  const int64_t row0 = a.q_cu[seq];
-  const int n = a.q_cu[seq + 1] - (int)row0;
-  const int64_t pr0 = row0 - a.n_single;
-  const int p0 = a.positions[row0];
-  const int slot = a.state_slots[seq];
-  const int qh = head / (a.heads / a.qk_heads);
-  const int rg = lane & 15;
-  const int col_wg = 4 * CPL * wave + CPL * (lane >> 4);   // first column of this lane in the workgroup
-  const int col = cb * COLS + col_wg;
-  float* S = a.state + ((int64_t)slot * a.heads + head) * DK * a.v_pad;
+  const int head = blockIdx.x % a.heads;
+  const int64_t chunk = blockIdx.x / a.heads;
+  const int32_t* cd = a.chunks + 3 * chunk;
+  const int seq = cd[0], n = cd[2];
+  const int64_t row = cd[1], row0 = a.q_cu[seq];
+  const int p = a.positions[row];
+  const int qh = head / (a.heads / a.qk_heads), qk = a.qk_heads * a.dim;
+  const ChunkRecord<DK> at{a.v_pad};
+  float* rec = a.pre + (chunk * a.heads + head) * at.size();
+  const E* ring = nullptr;
+  if constexpr (DELTA)
+    ring = reinterpret_cast<const E*>(a.conv_ring) + (int64_t)a.state_slots[seq] * a.taps * (2 * (int64_t)qk + (int64_t)a.heads * a.vdim);
+  const E* in = reinterpret_cast<const E*>(a.proj) + row * a.ld_proj;
+  const float step_l = DELTA ? 0.f : fmaxf(log2f(a.decay[head]), -126.f);
 
-  float s[CPL][R];
-#pragma unroll
-  for (int c = 0; c < CPL; ++c)
-#pragma unroll
-    for (int r = 0; r < R; ++r) s[c][r] = p0 > 0 && col + c < a.v_pad ? S[(int64_t)row_of<R>(rg, r) * a.v_pad + col + c] : 0.f;
-
-  f32x4 stage[PER];
-  float stage_beta = 0.f;
-  auto load_chunk = [&](int t0) {
-#pragma unroll
-    for (int i = 0; i < PER; ++i) {
-      const int idx = tid + 256 * i, t = idx / (ROWF / 4), e = (idx % (ROWF / 4)) * 4;
-      const int64_t pr = pr0 + min(t0 + t, n - 1);
-      const float* src;
-      if (e < 2 * DK) src = a.pre_qk + (pr * a.qk_heads + qh) * 2 * DK + e;
-      else if (DELTA && e < 3 * DK) src = a.pre_g + (pr * a.heads + head) * DK + (e - 2 * DK);
-      else src = a.pre_v + (pr * a.heads + head) * a.v_pad + min(cb * COLS + (e - NV * DK), a.v_pad - 4);
-      stage[i] = idx < V4 ? *reinterpret_cast<const f32x4*>(src) : f32x4{0.f, 0.f, 0.f, 0.f};
-    }
-    if (DELTA && tid < TC) stage_beta = a.pre_beta[(pr0 + min(t0 + tid, n - 1)) * a.heads + head];
-  };
-  auto store_chunk = [&](int b) {
-#pragma unroll
-    for (int i = 0; i < PER; ++i)
-      if (tid + 256 * i < V4) *reinterpret_cast<f32x4*>(&buf[b][4 * (tid + 256 * i)]) = stage[i];
-    if (DELTA && tid < TC) sbeta[b][tid] = stage_beta;
-  };
-  const float d = DELTA ? 1.0f : a.decay[head];
-
-  load_chunk(0);
-  store_chunk(0);
-  __syncthreads();
-  for (int t0 = 0, b = 0; t0 < n; t0 += TC, b ^= 1) {
-    if (t0 + TC < n) load_chunk(t0 + TC);
-    const int m = min(TC, n - t0);
-    float keep[CPL];
-#pragma unroll
-    for (int c = 0; c < CPL; ++c) keep[c] = 0.f;
-    auto token = [&](int t) {
-      const float* x = &buf[b][t * ROWF];
-      float q[R], k[R], v[CPL];
-      load_rows<R>(x + DK, rg, k);
-#pragma unroll
-      for (int c = 0; c < CPL; ++c) v[c] = x[NV * DK + col_wg + c];
+  for (int i = tid; i < 16 * DK; i += 256) {
+    const int t = i / DK, c = i % DK;
+    float q = 0.f, k = 0.f, l = 0.f;
+    if (t < n && c < a.dim) {
       if constexpr (DELTA) {
-        float g[R];
-        load_rows<R>(x + 2 * DK, rg, g);
-        load_rows<R>(x, rg, q);
-        const float beta = sbeta[b][t];
+        q = conv_input<E>(a, ring, row + t, row0, p + t, qh * a.dim + c);
+        k = conv_input<E>(a, ring, row + t, row0, p + t, qk + qh * a.dim + c);
+        l = LOG2E_F * decay_exponent<E>(a, row + t, head, c);
+      } else {
+        q = silu_f32(to_f32(in[t * a.ld_proj + a.off_q + qh * a.dim + c]));
+        k = silu_f32(to_f32(in[t * a.ld_proj + a.off_k + qh * a.dim + c]));
+        l = step_l;
+      }
+    }
+    sq[t * LD + c] = q, sk[t * LD + c] = k, sL[t * LD + c] = l;
+  }
+  for (int i = tid; i < 16 * a.v_pad; i += 256) {
+    const int t = i / a.v_pad, c = i % a.v_pad;
+    float v = 0.f;
+    if (t < n && c < a.vdim) {
+      if constexpr (DELTA) v = conv_input<E>(a, ring, row + t, row0, p + t, 2 * qk + head * a.vdim + c);
+      else v = silu_f32(to_f32(in[t * a.ld_proj + a.off_v + head * a.vdim + c]));
+    }
+    rec[ChunkRecord<DK>::V + i] = v;
+  }
+  if (DELTA && tid < 16) sbeta[tid] = tid < n ? sigmoid_full(to_f32(in[tid * a.ld_proj + a.off_b + head])) : 0.f;
+  __syncthreads();
+  if constexpr (DELTA) {   // unit vectors: four tokens per wave
 #pragma unroll
-        for (int c = 0; c < CPL; ++c) {
-          float kv[2] = {0.f, 0.f};
+    for (int j = 0; j < 4; ++j) {
+      const int t = 4 * wave + j;
+      float nq = 0.f, nk = 0.f;
+      for (int c = lane; c < DK; c += 64) {
+        nq = __builtin_fmaf(sq[t * LD + c], sq[t * LD + c], nq);
+        nk = __builtin_fmaf(sk[t * LD + c], sk[t * LD + c], nk);
+      }
+      const float fq = a.q_scale / sqrtf(wave_sum(nq) + a.unit_eps), fk = 1.0f / sqrtf(wave_sum(nk) + a.unit_eps);
+      for (int c = lane; c < DK; c += 64) sq[t * LD + c] *= fq, sk[t * LD + c] *= fk;
+    }
+  }
+  if (tid < DK) {
+    float l = 0.f;
 #pragma unroll
-          for (int r = 0; r < R; ++r) {
-            s[c][r] *= g[r];
-            kv[r & 1] = __builtin_fmaf(k[r], s[c][r], kv[r & 1]);
-          }
-          v[c] = beta * (v[c] - group_sum<16>(kv[0] + kv[1]));
+    for (int t = 0; t < 16; ++t) {
+      l += sL[t * LD + tid];
+      sL[t * LD + tid] = l;
+    }
+  }
+  __syncthreads();
+  {
+    const int t = tid >> 4, s = tid & 15;
+    float x = 0.f, y = 0.f;
+    if (s <= t) {
+      if constexpr (DELTA) {
+#pragma unroll 4
+        for (int c = 0; c < DK; ++c) {
+          const float e = sk[s * LD + c] * fast_exp2(sL[t * LD + c] - sL[s * LD + c]);
+          x = __builtin_fmaf(sk[t * LD + c], e, x);
+          y = __builtin_fmaf(sq[t * LD + c], e, y);
         }
       } else {
-        load_rows<R>(x, rg, q);
-#pragma unroll
-        for (int c = 0; c < CPL; ++c)
-#pragma unroll
-          for (int r = 0; r < R; ++r) s[c][r] *= d;
-      }
-#pragma unroll
-      for (int c = 0; c < CPL; ++c) {
-        float o[2] = {0.f, 0.f};
-#pragma unroll
-        for (int r = 0; r < R; ++r) {
-          s[c][r] = __builtin_fmaf(k[r], v[c], s[c][r]);
-          o[r & 1] = __builtin_fmaf(q[r], s[c][r], o[r & 1]);
-        }
-        const float sum = group_sum<16>(o[0] + o[1]);
-        keep[c] = rg == t ? sum : keep[c];
-      }
-    };
-    if (m == TC) {
 #pragma unroll 4
-      for (int t = 0; t < TC; ++t) token(t);
-    } else {
-      for (int t = 0; t < m; ++t) token(t);
+        for (int c = 0; c < DK; ++c) y = __builtin_fmaf(sq[t * LD + c], sk[s * LD + c], y);
+        y *= fast_exp2(sL[t * LD] - sL[s * LD]);
+      }
     }
-    if (rg < m)
-#pragma unroll
-      for (int c = 0; c < CPL; ++c)
-        if (col + c < a.v_pad) a.o[((pr0 + t0 + rg) * a.heads + head) * a.v_pad + col + c] = keep[c];
-    if (t0 + TC < n) store_chunk(b ^ 1);
+    rec[at.b() + tid] = y;
+    sa[t][s] = x;
+  }
+  for (int i = tid; i < 16 * DK; i += 256) {
+    const int t = i / DK, c = i % DK;
+    const float e = fast_exp2(sL[t * LD + c]);
+    if constexpr (DELTA) rec[ChunkRecord<DK>::KD + i] = sk[t * LD + c] * e;
+    rec[ChunkRecord<DK>::QD + i] = sq[t * LD + c] * e;
+    const int u = i & 15, d = i >> 4;
+    rec[ChunkRecord<DK>::KR + i] = sk[u * LD + d] * fast_exp2(sL[15 * LD + d] - sL[u * LD + d]);
+  }
+  if (tid < DK) rec[ChunkRecord<DK>::GE + tid] = fast_exp2(sL[15 * LD + tid]);
+  if constexpr (DELTA) {
     __syncthreads();
+    if (tid < 16) {   // column tid of T by forward substitution
+      float x[16];
+#pragma unroll
+      for (int t = 0; t < 16; ++t) {
+        float v = t == tid ? 1.0f : 0.f;
+#pragma unroll
+        for (int s = 0; s < t; ++s) v = __builtin_fmaf(-sa[t][s], x[s], v);
+        x[t] = sbeta[t] * v;
+        rec[at.t() + 16 * t + tid] = x[t];
+      }
+    }
+  }
+}
+
+// One workgroup per (sequence, head, 16 columns of S), chunk after chunk.  Its waves share the key channels: a wave keeps
+// TPW tiles [16 x 16] of S in registers in the accumulator layout of the 32-bit MFMA (row 4 g + r, column l16), which is the
+// layout its right operand takes when the contraction index of product r is 4 g + r.  Partial products with S0 meet in
+// LDS, one barrier a chunk; U is computed by every wave.  The next chunk's operands travel meanwhile.
+template <int TPW>
+struct ChunkOperands {
+  f32x4 kd[TPW], qd[TPW], kr[TPW], ge[TPW], t, b, v;
+};
+
+template <typename E, int MODE, int DK, int W>
+__global__ void __launch_bounds__(64 * W) recurrent_scan_kernel(const slm_recurrent_args a) {
+  constexpr bool DELTA = DELTA_MODE(MODE);
+  constexpr int TPW = DK / 16 / W;
+  __shared__ f32x4 part[2][2][W][64];
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int l16 = lane & 15, g = lane >> 4;
+  // the column blocks of one head on one XCD (workgroups go round the XCDs): they read the same records
+  const int n_cb = a.v_pad / 16, n_items = (a.batch - a.n_single) * a.heads;
+  const int cb = blockIdx.x / 8 % n_cb, item = blockIdx.x / (8 * n_cb) * 8 + blockIdx.x % 8;
+  if (item >= n_items) return;
+  const int head = item % a.heads, ps = item / a.heads, seq = a.n_single + ps;
+  const int64_t row0 = a.q_cu[seq];
+  const int n = a.q_cu[seq + 1] - (int)row0;
+  const int p0 = a.positions[row0], slot = a.state_slots[seq];
+  const int64_t chunk0 = a.seq_chunks[ps];
+  const int n_chunks = (n + 15) / 16;
+  const ChunkRecord<DK> at{a.v_pad};
+  const float* rec0 = a.pre + (chunk0 * a.heads + head) * at.size();
+  const int64_t rec_step = a.heads * at.size();
+  float* S = a.state + (((int64_t)slot * a.heads + head) * DK + 16 * TPW * wave + 4 * g) * a.v_pad + 16 * cb + l16;
+
+  f32x4 s[TPW];
+#pragma unroll
+  for (int i = 0; i < TPW; ++i)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) s[i][r] = p0 > 0 ? S[(int64_t)(16 * i + r) * a.v_pad] : 0.f;
+
+  auto load = [&](int c, ChunkOperands<TPW>& x) {
+    const float* rec = rec0 + c * rec_step;
+#pragma unroll
+    for (int i = 0; i < TPW; ++i) {
+      const int d = 16 * (TPW * wave + i);
+      if constexpr (DELTA) x.kd[i] = *reinterpret_cast<const f32x4*>(rec + ChunkRecord<DK>::KD + l16 * DK + d + 4 * g);
+      x.qd[i] = *reinterpret_cast<const f32x4*>(rec + ChunkRecord<DK>::QD + l16 * DK + d + 4 * g);
+      x.kr[i] = *reinterpret_cast<const f32x4*>(rec + ChunkRecord<DK>::KR + (d + l16) * 16 + 4 * g);
+      x.ge[i] = *reinterpret_cast<const f32x4*>(rec + ChunkRecord<DK>::GE + d + 4 * g);
+    }
+    if constexpr (DELTA) x.t = *reinterpret_cast<const f32x4*>(rec + at.t() + l16 * 16 + 4 * g);
+    x.b = *reinterpret_cast<const f32x4*>(rec + at.b() + l16 * 16 + 4 * g);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) x.v[r] = rec[ChunkRecord<DK>::V + (4 * g + r) * a.v_pad + 16 * cb + l16];
+  };
+  auto mma4 = [](const f32x4& x, const f32x4& y, f32x4 c) {
+#pragma unroll
+    for (int r = 0; r < 4; ++r) c = __builtin_amdgcn_mfma_f32_16x16x4f32(x[r], y[r], c, 0, 0, 0);
+    return c;
+  };
+  auto chunk = [&](int c, const ChunkOperands<TPW>& x) {
+    const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+    const int b = c & 1;
+    f32x4 kr = zero, o = zero;
+#pragma unroll
+    for (int i = 0; i < TPW; ++i) {
+      if constexpr (DELTA) kr = mma4(x.kd[i], s[i], kr);
+      o = mma4(x.qd[i], s[i], o);
+    }
+    if constexpr (DELTA) part[b][0][wave][lane] = kr;
+    part[b][1][wave][lane] = o;
+    lds_barrier();
+    f32x4 u = x.v;
+    if constexpr (DELTA) {
+#pragma unroll
+      for (int w = 0; w < W; ++w) u -= part[b][0][w][lane];
+      u = mma4(x.t, u, zero);
+    }
+#pragma unroll
+    for (int i = 0; i < TPW; ++i) s[i] = mma4(x.kr[i], u, s[i] * x.ge[i]);
+    if (c % W == wave) {   // (the waves take the outputs in turn)
+      o = part[b][1][0][lane];
+#pragma unroll
+      for (int w = 1; w < W; ++w) o += part[b][1][w][lane];
+      o = mma4(x.b, u, o);
+      float* dst = a.o + ((row0 - a.n_single + 16 * c + 4 * g) * a.heads + head) * a.v_pad + 16 * cb + l16;
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        if (16 * c + 4 * g + r < n) dst[(int64_t)r * a.heads * a.v_pad] = o[r];
+    }
+  };
+  ChunkOperands<TPW> x, y;
+  load(0, x);
+  for (int c = 0; c < n_chunks; c += 2) {
+    load(min(c + 1, n_chunks - 1), y);
+    chunk(c, x);
+    if (c + 1 >= n_chunks) break;
+    load(min(c + 2, n_chunks - 1), x);
+    chunk(c + 1, y);
   }
 #pragma unroll
-  for (int c = 0; c < CPL; ++c)
-    if (col + c < a.v_pad)
+  for (int i = 0; i < TPW; ++i)
 #pragma unroll
-      for (int r = 0; r < R; ++r) S[(int64_t)row_of<R>(rg, r) * a.v_pad + col + c] = s[c][r];
+    for (int r = 0; r < 4; ++r) S[(int64_t)(16 * i + r) * a.v_pad] = s[i][r];
 
   // the last inputs of the convolutions (their readers ran in the launch before)
   if (DELTA && cb == 0) {
-    const int qk = a.qk_heads * a.dim;
+    const int qh = head / (a.heads / a.qk_heads), qk = a.qk_heads * a.dim;
     const int64_t ch = 2 * (int64_t)qk + (int64_t)a.heads * a.vdim;
     E* ring = reinterpret_cast<E*>(a.conv_ring) + (int64_t)slot * a.taps * ch;
     const bool first_of_group = head % (a.heads / a.qk_heads) == 0;
     for (int j = max(0, n - a.taps); j < n; ++j) {
       E* dst = ring + (int64_t)((p0 + j) % a.taps) * ch;
       if (first_of_group)
-        for (int i = tid; i < a.dim; i += 256) {
+        for (int i = tid; i < a.dim; i += 64 * W) {
           dst[qh * a.dim + i] = raw_input<E>(a, row0 + j, qh * a.dim + i);
           dst[qk + qh * a.dim + i] = raw_input<E>(a, row0 + j, qk + qh * a.dim + i);
         }
-      for (int i = tid; i < a.vdim; i += 256) dst[2 * qk + head * a.vdim + i] = raw_input<E>(a, row0 + j, 2 * qk + head * a.vdim + i);
+      for (int i = tid; i < a.vdim; i += 64 * W) dst[2 * qk + head * a.vdim + i] = raw_input<E>(a, row0 + j, 2 * qk + head * a.vdim + i);
     }
   }
 }
@@ -498,32 +538,35 @@ static int rec_step(const slm_recurrent_args& a, hipStream_t st) {
   }
   return hip_check_launch();
 }
-template <typename E, int MODE, int R>
-static void rec_scan_r(const slm_recurrent_args& a, hipStream_t st) {
+template <typename E, int MODE, int DK>
+static void rec_scan_dk(const slm_recurrent_args& a, hipStream_t st) {
+  constexpr int W = DK / 16 < 4 ? DK / 16 : 4;
   const int64_t items = (int64_t)(a.batch - a.n_single) * a.heads;
-  // two columns per lane read the staged rows half as often: where enough workgroups are left to fill the chip
-  if (R <= 8 && items * ((a.v_pad + 31) / 32) >= 512)
-    recurrent_scan_kernel<E, MODE, R, (R <= 8 ? 2 : 1)><<<dim3((unsigned)(items * ((a.v_pad + 31) / 32))), dim3(256), 0, st>>>(a);
-  else
-    recurrent_scan_kernel<E, MODE, R, 1><<<dim3((unsigned)(items * ((a.v_pad + 15) / 16))), dim3(256), 0, st>>>(a);
+  recurrent_scan_kernel<E, MODE, DK, W><<<dim3((unsigned)((items + 7) / 8 * 8 * (a.v_pad / 16))), dim3(64 * W), 0, st>>>(a);
 }
 template <typename E, int MODE>
 static int rec_scan(const slm_recurrent_args& a, hipStream_t st) {
   hip_clear_error();
-  switch (a.dim_pad / 16) {
-    case 2: rec_scan_r<E, MODE, 2>(a, st); break;
-    case 4: rec_scan_r<E, MODE, 4>(a, st); break;
-    case 8: rec_scan_r<E, MODE, 8>(a, st); break;
-    case 12: rec_scan_r<E, MODE, 12>(a, st); break;
-    default: rec_scan_r<E, MODE, 16>(a, st);
+  switch (a.dim_pad) {
+    case 32: rec_scan_dk<E, MODE, 32>(a, st); break;
+    case 64: rec_scan_dk<E, MODE, 64>(a, st); break;
+    case 128: rec_scan_dk<E, MODE, 128>(a, st); break;
+    case 192: rec_scan_dk<E, MODE, 192>(a, st); break;
+    default: rec_scan_dk<E, MODE, 256>(a, st);
   }
   return hip_check_launch();
 }
 template <typename E, int MODE>
 static int rec_prepare(const slm_recurrent_args& a, hipStream_t st) {
-  const int n_tasks = 2 * a.qk_heads + (MODE == SLM_REC_DELTA ? 2 : 1) * a.heads;
+  const dim3 grid((unsigned)((int64_t)a.n_chunks * a.heads)), block(256);
   hip_clear_error();
-  recurrent_prepare_kernel<E, MODE><<<dim3((unsigned)(a.rows - a.n_single), (unsigned)((n_tasks + 3) / 4)), dim3(256), 0, st>>>(a);
+  switch (a.dim_pad) {
+    case 32: recurrent_prepare_kernel<E, MODE, 32><<<grid, block, 0, st>>>(a); break;
+    case 64: recurrent_prepare_kernel<E, MODE, 64><<<grid, block, 0, st>>>(a); break;
+    case 128: recurrent_prepare_kernel<E, MODE, 128><<<grid, block, 0, st>>>(a); break;
+    case 192: recurrent_prepare_kernel<E, MODE, 192><<<grid, block, 0, st>>>(a); break;
+    default: recurrent_prepare_kernel<E, MODE, 256><<<grid, block, 0, st>>>(a);
+  }
   return hip_check_launch();
 }
 
@@ -548,16 +591,19 @@ extern "C" SLM_API int slm_recurrent_step(const slm_recurrent_args* a, void* str
   if (a->n_single == 0) return SLM_OK;
   SLM_REC_DISPATCH(rec_step)
 }
+static bool rec_chunks_ok(const slm_recurrent_args& a) {
+  return a.pre && a.chunks && a.seq_chunks && a.n_chunks >= 0 && (int64_t)a.n_chunks * a.heads <= 0x7fffffff;
+}
+extern "C" SLM_API int64_t slm_recurrent_record_floats(int32_t dim_pad, int32_t v_pad) { return 49 * (int64_t)dim_pad + 16 * (int64_t)v_pad + 512; }
 extern "C" SLM_API int slm_recurrent_prepare(const slm_recurrent_args* a, void* stream) {
-  if (!a || !rec_sizes_ok(*a) || !rec_ptrs_ok(*a) || !a->pre_qk || !a->pre_v) return SLM_ERR_INVALID_ARG;
-  if (a->mode == SLM_REC_DELTA && (!a->pre_g || !a->pre_beta)) return SLM_ERR_INVALID_ARG;
-  if (a->rows == a->n_single) return SLM_OK;
+  if (!a || !rec_sizes_ok(*a) || !rec_ptrs_ok(*a) || !rec_chunks_ok(*a)) return SLM_ERR_INVALID_ARG;
+  if (!aligned16(a->pre)) return SLM_ERR_ALIGNMENT;
+  if (a->n_chunks == 0) return SLM_OK;
   SLM_REC_DISPATCH(rec_prepare)
 }
 extern "C" SLM_API int slm_recurrent_scan(const slm_recurrent_args* a, void* stream) {
-  if (!a || !rec_sizes_ok(*a) || !rec_ptrs_ok(*a) || !a->pre_qk || !a->pre_v || !a->o) return SLM_ERR_INVALID_ARG;
-  if (a->mode == SLM_REC_DELTA && (!a->pre_g || !a->pre_beta)) return SLM_ERR_INVALID_ARG;
-  if (!aligned16(a->pre_qk) || !aligned16(a->pre_v) || !aligned16(a->pre_g)) return SLM_ERR_ALIGNMENT;
+  if (!a || !rec_sizes_ok(*a) || !rec_ptrs_ok(*a) || !rec_chunks_ok(*a) || !a->o) return SLM_ERR_INVALID_ARG;
+  if (!aligned16(a->pre)) return SLM_ERR_ALIGNMENT;
   if (a->batch == a->n_single) return SLM_OK;
   SLM_REC_DISPATCH(rec_scan)
 }

@@ -9,13 +9,14 @@ import ctypes as C
 from dataclasses import dataclass
 from typing import Optional
 
+import numpy as np
 import torch
 
 from . import _lib
 from ._lib import mixers_check
 from .kernels import reserve_workspace
 from .latent_kernels import _code, _i32, _need, _p, _stream
-from .layers import RecurrentState
+from .layers import InputParameters, RecurrentState
 
 
 def recurrent_dim_pad(dim: int) -> int:
@@ -120,21 +121,43 @@ def recurrent_step(s: RecurrentSpec, proj: torch.Tensor, low: Optional[torch.Ten
     return o
 
 
+@dataclass
+class ChunkPlan:
+    """The portions of a step in chunks of at most 16 tokens (see slm_recurrent_args)."""
+    CHUNK = 16
+    chunks: torch.Tensor       # [n_chunks, 3] int32: sequence, first row, rows
+    seq_chunks: torch.Tensor   # [portions] int32: first chunk
+
+    @staticmethod
+    def host(portions, n_single: int):
+        chunks, first = [], []
+        for i, p in enumerate(portions):
+            first.append(len(chunks))
+            chunks += [(n_single + i, p.row0 + t, min(ChunkPlan.CHUNK, p.q_len - t)) for t in range(0, p.q_len, ChunkPlan.CHUNK)]
+        return np.array(chunks, dtype=np.int32), np.array(first, dtype=np.int32)
+
+    @staticmethod
+    def of(params: InputParameters, n_single: int, device) -> "ChunkPlan":
+        plan = params.plans.get("chunks")
+        if plan is None:
+            chunks, first = ChunkPlan.host(params.portions, n_single)
+            plan = params.plans["chunks"] = ChunkPlan(torch.from_numpy(chunks).to(device), torch.from_numpy(first).to(device))
+        return plan
+
+
 def recurrent_portions(s: RecurrentSpec, proj: torch.Tensor, low: Optional[torch.Tensor], state: RecurrentState,
-                       positions: torch.Tensor, q_cu: torch.Tensor, state_slots: torch.Tensor, n_single: int) -> torch.Tensor:
-    """The sequences behind the first n_single, token after token: read-outs [portion rows, heads, v_pad] fp32."""
+                       positions: torch.Tensor, q_cu: torch.Tensor, state_slots: torch.Tensor, n_single: int, plan: ChunkPlan) -> torch.Tensor:
+    """The sequences behind the first n_single, chunk after chunk: read-outs [portion rows, heads, v_pad] fp32."""
     a = _recurrent_args(s, proj, low, state, positions, q_cu, state_slots, n_single)
-    n, dev = proj.size(0) - n_single, proj.device
-    f32 = dict(dtype=torch.float32, device=dev)
-    o = torch.empty(n, s.heads, s.v_pad, **f32)
-    qk = torch.empty(n, s.qk_heads, 2, s.dim_pad, **f32)
-    v = torch.empty(n, s.heads, s.v_pad, **f32)
-    a.pre_qk, a.pre_v, a.o = _p(qk), _p(v), _p(o)
-    if s.mode == _lib.REC_DELTA:
-        g, beta = torch.empty(n, s.heads, s.dim_pad, **f32), torch.empty(n, s.heads, **f32)
-        a.pre_g, a.pre_beta = _p(g), _p(beta)
+    n, n_chunks, dev = proj.size(0) - n_single, plan.chunks.size(0), proj.device
+    L = _lib.mixers_lib()
+    o = torch.empty(n, s.heads, s.v_pad, dtype=torch.float32, device=dev)
+    pre = torch.empty(n_chunks, s.heads, L.slm_recurrent_record_floats(s.dim_pad, s.v_pad), dtype=torch.float32, device=dev)
+    _need(plan.chunks.dim() == 2 and plan.chunks.size(1) == 3 and n_chunks * ChunkPlan.CHUNK >= n, "recurrent: chunks")
+    _i32(plan.chunks, 3 * n_chunks, "chunks")
+    _i32(plan.seq_chunks, q_cu.numel() - 1 - n_single, "seq_chunks")
+    a.chunks, a.seq_chunks, a.n_chunks, a.pre, a.o = _p(plan.chunks), _p(plan.seq_chunks), n_chunks, _p(pre), _p(o)
     if n:
-        L = _lib.mixers_lib()
         mixers_check(L.slm_recurrent_prepare(C.byref(a), _stream()), "slm_recurrent_prepare")
         mixers_check(L.slm_recurrent_scan(C.byref(a), _stream()), "slm_recurrent_scan")
     return o

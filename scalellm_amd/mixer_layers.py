@@ -192,7 +192,7 @@ class LightningAttention:
         if n:
             mk.gated_norm(mk.recurrent_step(*step), self.args.vdim, gate[:n], self.norm, out[:n], **how)
         if n < proj.size(0):
-            mk.gated_norm(mk.recurrent_portions(*step), self.args.vdim, gate[n:], self.norm, out[n:], **how)
+            mk.gated_norm(mk.recurrent_portions(*step, mk.ChunkPlan.of(params, n, proj.device)), self.args.vdim, gate[n:], self.norm, out[n:], **how)
 
 
 # ---------------------------------------------------------------------------------------
@@ -289,5 +289,5 @@ class ChannelDelta:
         if n:
             mk.recurrent_step(*step, out=out[:n])
         if n < T:
-            mk.gated_norm(mk.recurrent_portions(*step), s.vdim, low[n:, self.low_n:], s.norm_weight, out[n:], eps=self.eps, per_head=True)
+            mk.gated_norm(mk.recurrent_portions(*step, mk.ChunkPlan.of(params, n, proj.device)), s.vdim, low[n:, self.low_n:], s.norm_weight, out[n:], eps=self.eps, per_head=True)
         return out_product(out, self.w_o)

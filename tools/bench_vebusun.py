@@ -25,7 +25,7 @@ from scalellm_amd.registry import ModelLimits  # noqa: E402
 from scalellm_amd.vebusun import VebusunStep  # noqa: E402
 from tools.bench_dagupel import BLOCK, DEV, HBM, MFMA, SIZES, RandomCheckpoint, batch, dagupel, llama, timed, visible_pairs  # noqa: E402
 
-VALU = 78.6e12   # fp32 fused multiply-adds without packed arithmetic
+FP32 = 157.3e12   # 32-bit matrix products
 KEEP = 16
 
 
@@ -104,10 +104,10 @@ def main(argv=None):
                  llama(size, L, need * (BLOCK // 16), most))
             base = dict(size=size, model=which, layers=L)
 
-            def kernel(name, fn, count, nbytes=0, flops=0, valu=0, **rec):
+            def kernel(name, fn, count, nbytes=0, flops=0, fp32=0, **rec):
                 t = timed(fn) / count
-                roof = max(nbytes / HBM, flops / MFMA, valu / VALU)
-                emit(kind="kernel", **base, kernel=name, us=t * 1e6, tb_per_s=nbytes / t / 1e12, tflops=(flops + valu) / t / 1e12,
+                roof = max(nbytes / HBM, flops / MFMA, fp32 / FP32)
+                emit(kind="kernel", **base, kernel=name, us=t * 1e6, tb_per_s=nbytes / t / 1e12, tflops=(flops + fp32) / t / 1e12,
                      roofline=roof / t, **rec)
             if V:
                 pairs = list(zip(m.layers, m.caches))
@@ -115,6 +115,7 @@ def main(argv=None):
                 paras = [(x, c) for x, c in pairs if not isinstance(x.mixer, ChannelDelta)]
                 d0, p0 = deltas[0][0].mixer, paras[0][0].mixer
                 S = heads * 128 * 128
+                chunk_flops = 3 * 2 * S + 2 * heads * (2 * 16 * 128 + 2 * 16 * 128)
             for bs in sizes:
                 context = args.context if which != "llama" else min(args.context, window)
                 tokens, positions, params, _ = make_decode_inputs(bs, context, block, DEV, seed=1, vocab=vocab)
@@ -174,13 +175,14 @@ def main(argv=None):
                 low = torch.randn(T, 2 * d0.low_n, device=DEV).to(torch.bfloat16)
                 out = torch.empty(T, max(p0.o_k, d0.o_k), device=DEV, dtype=torch.bfloat16)
                 step = (positions, params.q_cu_seq_lens, params.state_slots, 0)
+                chunks = mk.ChunkPlan.of(params, 0, DEV)
                 x, c = deltas[0]
-                # what a token costs: S * g, k.S, S + k u, q.S
-                kernel("delta portions (prepare + scan)", lambda: mk.recurrent_portions(x.mixer.spec, projd, low, c, *step), 1, valu=T * S * 7,
+                # 32-bit products of a token in chunks of 16: three with the state, four 16 wide
+                kernel("delta portions (prepare + scan)", lambda: mk.recurrent_portions(x.mixer.spec, projd, low, c, *step, chunks), 1, fp32=T * chunk_flops,
                        nbytes=T * heads * 128 * (8 + 4 * 8), batch=name)
                 y, e = paras[0]
-                kernel("lightning portions (prepare + scan)", lambda: mk.recurrent_portions(y.mixer.right.spec, projp[:, p0.split:], None, e[1], *step), 1,
-                       valu=T * S * 5, nbytes=T * heads * 128 * (6 + 4 * 6), batch=name)
+                kernel("lightning portions (prepare + scan)", lambda: mk.recurrent_portions(y.mixer.right.spec, projp[:, p0.split:], None, e[1], *step, chunks), 1,
+                       fp32=T * (chunk_flops - 2 * S - 2 * heads * 2 * 16 * 128), nbytes=T * heads * 128 * (6 + 4 * 6), batch=name)
                 o = torch.randn(T, heads, 128, device=DEV)
                 kernel("norm + gate", lambda: mk.gated_norm(o, 128, low[:, d0.low_n:], d0.spec.norm_weight, out[:, :d0.o_k], eps=1e-5, per_head=True), 1,
                        nbytes=T * heads * 128 * 8, batch=name)
