@@ -16,7 +16,12 @@ namespace slm {
 constexpr bool DELTA_MODE(int m) { return m == SLM_REC_DELTA; }
 
 __device__ __forceinline__ float silu_f32(float z) { return z / (1.0f + __expf(-z)); }
-__device__ __forceinline__ float softplus_f32(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+// log(1 + x) = log(u) x / (u - 1) with u the rounded 1 + x: what the sum loses of x comes back (Kahan)
+__device__ __forceinline__ float softplus_f32(float z) {
+  const float x = __expf(-fabsf(z)), u = 1.0f + x;
+  const float l = u == 1.0f ? x : __logf(u) * (x / (u - 1.0f));
+  return fmaxf(z, 0.f) + l;
+}
 __device__ __forceinline__ float sigmoid_full(float z) { return 1.0f / (1.0f + expf(-z)); }
 
 // the convolved, activated input of channel c (index into q | k | v) of `row` at position p; rows of the step before
@@ -40,6 +45,32 @@ __device__ __forceinline__ E raw_input(const slm_recurrent_args& a, int64_t row,
   const int qk = a.qk_heads * a.dim;
   const int64_t col = c < qk ? a.off_q + c : c < 2 * qk ? a.off_k + (c - qk) : a.off_v + (c - 2 * qk);
   return reinterpret_cast<const E*>(a.proj)[row * a.ld_proj + col];
+}
+// the same for the 16 tokens from `row` on (n of them there are), convolutions of at most 4 taps: every input is read once
+template <typename E, typename F>
+__device__ __forceinline__ void conv_run4(const slm_recurrent_args& a, const E* ring, int64_t row, int64_t row0, int p, int n, int c, F put) {
+  const int64_t ch = 2 * (int64_t)a.qk_heads * a.dim + (int64_t)a.heads * a.vdim;
+  const int qk = a.qk_heads * a.dim;
+  const int64_t col = c < qk ? a.off_q + c : c < 2 * qk ? a.off_k + (c - qk) : a.off_v + (c - 2 * qk);
+  const E* src = reinterpret_cast<const E*>(a.proj) + row * a.ld_proj + col;
+  float w[4], x[19];   // w[j]: of the input j tokens back; x[3 + t]: the input of token t
+#pragma unroll
+  for (int j = 0; j < 4; ++j) w[j] = j < a.taps ? a.conv_w[(int64_t)(a.taps - 1 - j) * ch + c] : 0.f;
+#pragma unroll
+  for (int j = 1; j < 4; ++j) {
+    x[3 - j] = 0.f;
+    if (j < a.taps && p >= j)
+      x[3 - j] = row - j >= row0 ? to_f32(src[-j * a.ld_proj]) : to_f32(ring[(int64_t)((p - j) % a.taps) * ch + c]);
+  }
+#pragma unroll
+  for (int t = 0; t < 16; ++t) x[3 + t] = to_f32(src[min(t, n - 1) * a.ld_proj]);
+#pragma unroll
+  for (int t = 0; t < 16; ++t) {
+    float acc = w[3] * x[t];
+#pragma unroll
+    for (int j = 2; j >= 0; --j) acc = __builtin_fmaf(w[j], x[3 + t - j], acc);
+    put(t, t < n ? silu_f32(acc) : 0.f);
+  }
 }
 template <typename E>
 __device__ __forceinline__ float decay_exponent(const slm_recurrent_args& a, int64_t row, int head, int c) {
@@ -240,8 +271,9 @@ struct ChunkRecord {
 template <typename E, int MODE, int DK>
 __global__ void __launch_bounds__(256) recurrent_prepare_kernel(const slm_recurrent_args a) {
   constexpr bool DELTA = DELTA_MODE(MODE);
-  constexpr int LD = DK + 1;                     // (odd: the 16 rows a half-wave reads are in different banks)
-  __shared__ float sq[16 * LD], sk[16 * LD], sL[16 * LD], sa[16][17], sbeta[16];
+  constexpr int LD = DK + 4;                     // (the 16 rows a quarter-wave reads by 16 bytes are in different banks)
+  __shared__ __attribute__((aligned(16))) float sq[16 * LD], sk[16 * LD], sL[16 * LD];
+  __shared__ float sa[16][17], sbeta[16];
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int head = blockIdx.x % a.heads;
   const int64_t chunk = blockIdx.x / a.heads;
@@ -258,30 +290,63 @@ __global__ void __launch_bounds__(256) recurrent_prepare_kernel(const slm_recurr
   const E* in = reinterpret_cast<const E*>(a.proj) + row * a.ld_proj;
   const float step_l = DELTA ? 0.f : fmaxf(log2f(a.decay[head]), -126.f);
 
-  for (int i = tid; i < 16 * DK; i += 256) {
-    const int t = i / DK, c = i % DK;
-    float q = 0.f, k = 0.f, l = 0.f;
-    if (t < n && c < a.dim) {
-      if constexpr (DELTA) {
-        q = conv_input<E>(a, ring, row + t, row0, p + t, qh * a.dim + c);
-        k = conv_input<E>(a, ring, row + t, row0, p + t, qk + qh * a.dim + c);
-        l = LOG2E_F * decay_exponent<E>(a, row + t, head, c);
+  if (DELTA && a.taps <= 4) {
+    for (int i = tid; i < 2 * DK + a.v_pad; i += 256) {
+      if (i < 2 * DK) {
+        const int c = i < DK ? i : i - DK;
+        float* dst = (i < DK ? sq : sk) + c;
+        auto put = [&](int t, float x) { dst[t * LD] = x; };
+        if (c < a.dim) {
+          conv_run4<E>(a, ring, row, row0, p, n, (i < DK ? 0 : qk) + qh * a.dim + c, put);
+        } else {
+#pragma unroll
+          for (int t = 0; t < 16; ++t) put(t, 0.f);
+        }
       } else {
-        q = silu_f32(to_f32(in[t * a.ld_proj + a.off_q + qh * a.dim + c]));
-        k = silu_f32(to_f32(in[t * a.ld_proj + a.off_k + qh * a.dim + c]));
-        l = step_l;
+        const int c = i - 2 * DK;
+        float* dst = rec + ChunkRecord<DK>::V + c;
+        auto put = [&](int t, float x) { dst[t * a.v_pad] = x; };
+        if (c < a.vdim) {
+          conv_run4<E>(a, ring, row, row0, p, n, 2 * qk + head * a.vdim + c, put);
+        } else {
+#pragma unroll
+          for (int t = 0; t < 16; ++t) put(t, 0.f);
+        }
       }
     }
-    sq[t * LD + c] = q, sk[t * LD + c] = k, sL[t * LD + c] = l;
-  }
-  for (int i = tid; i < 16 * a.v_pad; i += 256) {
-    const int t = i / a.v_pad, c = i % a.v_pad;
-    float v = 0.f;
-    if (t < n && c < a.vdim) {
-      if constexpr (DELTA) v = conv_input<E>(a, ring, row + t, row0, p + t, 2 * qk + head * a.vdim + c);
-      else v = silu_f32(to_f32(in[t * a.ld_proj + a.off_v + head * a.vdim + c]));
+  } else {
+    for (int i = tid; i < 16 * DK; i += 256) {
+      const int t = i / DK, c = i % DK;
+      float q = 0.f, k = 0.f;
+      if (t < n && c < a.dim) {
+        if constexpr (DELTA) {
+          q = conv_input<E>(a, ring, row + t, row0, p + t, qh * a.dim + c);
+          k = conv_input<E>(a, ring, row + t, row0, p + t, qk + qh * a.dim + c);
+        } else {
+          q = silu_f32(to_f32(in[t * a.ld_proj + a.off_q + qh * a.dim + c]));
+          k = silu_f32(to_f32(in[t * a.ld_proj + a.off_k + qh * a.dim + c]));
+        }
+      }
+      sq[t * LD + c] = q, sk[t * LD + c] = k;
     }
-    rec[ChunkRecord<DK>::V + i] = v;
+    for (int i = tid; i < 16 * a.v_pad; i += 256) {
+      const int t = i / a.v_pad, c = i % a.v_pad;
+      float v = 0.f;
+      if (t < n && c < a.vdim) {
+        if constexpr (DELTA) v = conv_input<E>(a, ring, row + t, row0, p + t, 2 * qk + head * a.vdim + c);
+        else v = silu_f32(to_f32(in[t * a.ld_proj + a.off_v + head * a.vdim + c]));
+      }
+      rec[ChunkRecord<DK>::V + i] = v;
+    }
+  }
+  for (int i = tid; i < 16 * DK; i += 256) {
+    const int t = i / DK, c = i % DK;
+    float l = 0.f;
+    if (t < n && c < a.dim) {
+      if constexpr (DELTA) l = LOG2E_F * decay_exponent<E>(a, row + t, head, c);
+      else l = step_l;
+    }
+    sL[t * LD + c] = l;
   }
   if (DELTA && tid < 16) sbeta[tid] = tid < n ? sigmoid_full(to_f32(in[tid * a.ld_proj + a.off_b + head])) : 0.f;
   __syncthreads();
@@ -312,28 +377,42 @@ __global__ void __launch_bounds__(256) recurrent_prepare_kernel(const slm_recurr
     float x = 0.f, y = 0.f;
     if (s <= t) {
       if constexpr (DELTA) {
-#pragma unroll 4
-        for (int c = 0; c < DK; ++c) {
-          const float e = sk[s * LD + c] * fast_exp2(sL[t * LD + c] - sL[s * LD + c]);
-          x = __builtin_fmaf(sk[t * LD + c], e, x);
-          y = __builtin_fmaf(sq[t * LD + c], e, y);
+#pragma unroll 2
+        for (int c = 0; c < DK; c += 4) {
+          const f32x4 ks = *reinterpret_cast<const f32x4*>(sk + s * LD + c), ls = *reinterpret_cast<const f32x4*>(sL + s * LD + c);
+          const f32x4 kt = *reinterpret_cast<const f32x4*>(sk + t * LD + c), lt = *reinterpret_cast<const f32x4*>(sL + t * LD + c);
+          const f32x4 qt = *reinterpret_cast<const f32x4*>(sq + t * LD + c);
+#pragma unroll
+          for (int j = 0; j < 4; ++j) {
+            const float e = ks[j] * fast_exp2(lt[j] - ls[j]);
+            x = __builtin_fmaf(kt[j], e, x);
+            y = __builtin_fmaf(qt[j], e, y);
+          }
         }
       } else {
-#pragma unroll 4
-        for (int c = 0; c < DK; ++c) y = __builtin_fmaf(sq[t * LD + c], sk[s * LD + c], y);
+#pragma unroll 2
+        for (int c = 0; c < DK; c += 4) {
+          const f32x4 ks = *reinterpret_cast<const f32x4*>(sk + s * LD + c), qt = *reinterpret_cast<const f32x4*>(sq + t * LD + c);
+#pragma unroll
+          for (int j = 0; j < 4; ++j) y = __builtin_fmaf(qt[j], ks[j], y);
+        }
         y *= fast_exp2(sL[t * LD] - sL[s * LD]);
       }
     }
     rec[at.b() + tid] = y;
     sa[t][s] = x;
   }
-  for (int i = tid; i < 16 * DK; i += 256) {
+  for (int i = 4 * tid; i < 16 * DK; i += 1024) {
     const int t = i / DK, c = i % DK;
-    const float e = fast_exp2(sL[t * LD + c]);
-    if constexpr (DELTA) rec[ChunkRecord<DK>::KD + i] = sk[t * LD + c] * e;
-    rec[ChunkRecord<DK>::QD + i] = sq[t * LD + c] * e;
+    const f32x4 l = *reinterpret_cast<const f32x4*>(sL + t * LD + c), q = *reinterpret_cast<const f32x4*>(sq + t * LD + c);
+    const f32x4 e = {fast_exp2(l.x), fast_exp2(l.y), fast_exp2(l.z), fast_exp2(l.w)};
+    if constexpr (DELTA) *reinterpret_cast<f32x4*>(rec + ChunkRecord<DK>::KD + i) = *reinterpret_cast<const f32x4*>(sk + t * LD + c) * e;
+    *reinterpret_cast<f32x4*>(rec + ChunkRecord<DK>::QD + i) = q * e;
     const int u = i & 15, d = i >> 4;
-    rec[ChunkRecord<DK>::KR + i] = sk[u * LD + d] * fast_exp2(sL[15 * LD + d] - sL[u * LD + d]);
+    f32x4 kr;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) kr[j] = sk[(u + j) * LD + d] * fast_exp2(sL[15 * LD + d] - sL[(u + j) * LD + d]);
+    *reinterpret_cast<f32x4*>(rec + ChunkRecord<DK>::KR + i) = kr;
   }
   if (tid < DK) rec[ChunkRecord<DK>::GE + tid] = fast_exp2(sL[15 * LD + tid]);
   if constexpr (DELTA) {
@@ -355,7 +434,8 @@ __global__ void __launch_bounds__(256) recurrent_prepare_kernel(const slm_recurr
 // One workgroup per (sequence, head, 16 columns of S), chunk after chunk.  Its waves share the key channels: a wave keeps
 // TPW tiles [16 x 16] of S in registers in the accumulator layout of the 32-bit MFMA (row 4 g + r, column l16), which is the
 // layout its right operand takes when the contraction index of product r is 4 g + r.  Partial products with S0 meet in
-// LDS, one barrier a chunk; U is computed by every wave.  The next chunk's operands travel meanwhile.
+// LDS, one barrier a chunk; U is computed by every wave.  The operands of the next chunks
+// travel meanwhile.
 template <int TPW>
 struct ChunkOperands {
   f32x4 kd[TPW], qd[TPW], kr[TPW], ge[TPW], t, b, v;
@@ -365,6 +445,7 @@ template <typename E, int MODE, int DK, int W>
 __global__ void __launch_bounds__(64 * W) recurrent_scan_kernel(const slm_recurrent_args a) {
   constexpr bool DELTA = DELTA_MODE(MODE);
   constexpr int TPW = DK / 16 / W;
+  constexpr int NB = TPW <= 2 ? 3 : 2;   // chunks in registers: one in use, the others on their way
   __shared__ f32x4 part[2][2][W][64];
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int l16 = lane & 15, g = lane >> 4;
@@ -440,14 +521,17 @@ __global__ void __launch_bounds__(64 * W) recurrent_scan_kernel(const slm_recurr
         if (16 * c + 4 * g + r < n) dst[(int64_t)r * a.heads * a.v_pad] = o[r];
     }
   };
-  ChunkOperands<TPW> x, y;
-  load(0, x);
-  for (int c = 0; c < n_chunks; c += 2) {
-    load(min(c + 1, n_chunks - 1), y);
-    chunk(c, x);
-    if (c + 1 >= n_chunks) break;
-    load(min(c + 2, n_chunks - 1), x);
-    chunk(c + 1, y);
+  ChunkOperands<TPW> x[NB];
+#pragma unroll
+  for (int i = 0; i + 1 < NB; ++i) load(min(i, n_chunks - 1), x[i]);
+  for (int c = 0; c < n_chunks; c += NB) {
+#pragma unroll
+    for (int i = 0; i < NB; ++i) {
+      if (c + i < n_chunks) {
+        load(min(c + i + NB - 1, n_chunks - 1), x[(i + NB - 1) % NB]);
+        chunk(c + i, x[i]);
+      }
+    }
   }
 #pragma unroll
   for (int i = 0; i < TPW; ++i)
