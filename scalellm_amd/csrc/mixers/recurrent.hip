@@ -442,7 +442,7 @@ struct ChunkOperands {
 };
 
 template <typename E, int MODE, int DK, int W>
-__global__ void __launch_bounds__(64 * W) recurrent_scan_kernel(const slm_recurrent_args a) {
+__global__ void __launch_bounds__(64 * W, 2) recurrent_scan_kernel(const slm_recurrent_args a) {
   constexpr bool DELTA = DELTA_MODE(MODE);
   constexpr int TPW = DK / 16 / W;
   constexpr int NB = TPW <= 2 ? 3 : 2;   // chunks in registers: one in use, the others on their way
@@ -524,15 +524,17 @@ __global__ void __launch_bounds__(64 * W) recurrent_scan_kernel(const slm_recurr
   ChunkOperands<TPW> x[NB];
 #pragma unroll
   for (int i = 0; i + 1 < NB; ++i) load(min(i, n_chunks - 1), x[i]);
-  for (int c = 0; c < n_chunks; c += NB) {
+  int c0 = 0;   // (whole rounds without a branch around the loads: a join would make every wait one for the youngest)
+  for (; c0 + NB <= n_chunks; c0 += NB) {
 #pragma unroll
     for (int i = 0; i < NB; ++i) {
-      if (c + i < n_chunks) {
-        load(min(c + i + NB - 1, n_chunks - 1), x[(i + NB - 1) % NB]);
-        chunk(c + i, x[i]);
-      }
+      load(min(c0 + i + NB - 1, n_chunks - 1), x[(i + NB - 1) % NB]);
+      chunk(c0 + i, x[i]);
     }
   }
+#pragma unroll
+  for (int i = 0; i + 1 < NB; ++i)
+    if (c0 + i < n_chunks) chunk(c0 + i, x[i]);
 #pragma unroll
   for (int i = 0; i < TPW; ++i)
 #pragma unroll
@@ -569,13 +571,20 @@ __global__ void __launch_bounds__(256) gated_norm_kernel(const slm_gated_norm_ar
     const int64_t row = item / a.heads;
     const int h = item % a.heads;
     const float* o = a.o + item * a.v_pad;
-    float ss = 0.f;
-    for (int c = lane; c < a.vdim; c += 64) ss = __builtin_fmaf(o[c], o[c], ss);
-    const float rs = 1.0f / sqrtf(wave_sum(ss) / (float)a.vdim + a.eps);
     const E* gate = reinterpret_cast<const E*>(a.gate) + row * a.ld_gate + (int64_t)h * a.vdim;
     E* out = reinterpret_cast<E*>(a.out) + row * a.ld_out;
-    for (int c = lane; c < a.vdim; c += 64)
-      out[h * a.vdim + c] = (E)(a.scale * o[c] * rs * a.weight[c] * sigmoid_f32(to_f32(gate[c])));
+    float x[4], gl[4], w[4], ss = 0.f;   // (v_pad <= 256)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int c = lane + 64 * j;
+      const bool in = c < a.vdim;
+      x[j] = in ? o[c] : 0.f, gl[j] = in ? to_f32(gate[c]) : 0.f, w[j] = in ? a.weight[c] : 0.f;
+      ss = __builtin_fmaf(x[j], x[j], ss);
+    }
+    const float rs = 1.0f / sqrtf(wave_sum(ss) / (float)a.vdim + a.eps);
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (lane + 64 * j < a.vdim) out[h * a.vdim + lane + 64 * j] = (E)(a.scale * x[j] * rs * w[j] * sigmoid_f32(gl[j]));
     if (h == a.heads - 1)
       for (int64_t c = (int64_t)a.heads * a.vdim + lane; c < a.out_width; c += 64) out[c] = (E)0.f;
   } else {
@@ -692,7 +701,7 @@ extern "C" SLM_API int slm_recurrent_scan(const slm_recurrent_args* a, void* str
   SLM_REC_DISPATCH(rec_scan)
 }
 extern "C" SLM_API int slm_gated_norm(const slm_gated_norm_args* a, void* stream) {
-  if (!a || !a->o || !a->gate || !a->weight || !a->out || a->rows < 0 || a->heads < 1 || a->vdim < 1 || a->v_pad < a->vdim ||
+  if (!a || !a->o || !a->gate || !a->weight || !a->out || a->rows < 0 || a->heads < 1 || a->vdim < 1 || a->v_pad < a->vdim || a->v_pad > 256 ||
       a->out_width < (int64_t)a->heads * a->vdim || a->ld_out < a->out_width || a->rows * a->heads > 0x7fffffff)
     return SLM_ERR_INVALID_ARG;
   if (a->dtype != SLM_BF16 && a->dtype != SLM_F32) return SLM_ERR_UNSUPPORTED;

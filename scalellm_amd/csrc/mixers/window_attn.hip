@@ -7,7 +7,7 @@ namespace slm {
 constexpr int WA_MAX = 512;   // widest head
 
 // one wave per (row, vector): q heads normed and rotated in place, k heads normed and rotated into the cache, v copied
-template <typename E>
+template <typename E, int NJ>   // NJ: columns per lane
 __global__ void __launch_bounds__(256) window_append_kernel(const slm_window_append_args a) {
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int64_t row = blockIdx.x;
@@ -29,9 +29,9 @@ __global__ void __launch_bounds__(256) window_append_kernel(const slm_window_app
   const int64_t p = min((int64_t)a.positions[row], a.max_positions - 1);
   const float* cs = a.cos_sin + p * a.rot;
   const int half = a.rot / 2;
-  float x[WA_MAX / 64], y[WA_MAX / 64], ss = 0.f;
+  float x[NJ], y[NJ], ss = 0.f;
 #pragma unroll
-  for (int j = 0; j < WA_MAX / 64; ++j) {
+  for (int j = 0; j < NJ; ++j) {
     const int c = lane + 64 * j;
     x[j] = y[j] = 0.f;
     if (c < a.dim) {
@@ -47,7 +47,7 @@ __global__ void __launch_bounds__(256) window_append_kernel(const slm_window_app
   const float rs = 1.0f / sqrtf(wave_sum(ss) / (float)a.dim + a.eps);
   E* dst = is_q ? src : reinterpret_cast<E*>(a.key_cache) + (slot * a.kv_heads + g) * a.d_pad;
 #pragma unroll
-  for (int j = 0; j < WA_MAX / 64; ++j) {
+  for (int j = 0; j < NJ; ++j) {
     const int c = lane + 64 * j;
     if (c >= a.d_pad) continue;
     float v = x[j] * rs;
@@ -134,6 +134,16 @@ __global__ void __launch_bounds__(256) window_attn_any_kernel(const slm_window_a
   }
 }
 
+template <typename E>
+static void append_launch(const slm_window_append_args& a, dim3 grid, hipStream_t st) {
+  switch ((a.d_pad + 63) / 64) {
+    case 1: window_append_kernel<E, 1><<<grid, dim3(256), 0, st>>>(a); break;
+    case 2: window_append_kernel<E, 2><<<grid, dim3(256), 0, st>>>(a); break;
+    case 3: case 4: window_append_kernel<E, 4><<<grid, dim3(256), 0, st>>>(a); break;
+    default: window_append_kernel<E, WA_MAX / 64><<<grid, dim3(256), 0, st>>>(a);
+  }
+}
+
 bool window_decode_ok(const slm_window_attn_args& a);
 size_t window_decode_workspace(const slm_window_attn_args& a);
 int window_decode(const slm_window_attn_args& a, hipStream_t st);
@@ -151,8 +161,8 @@ extern "C" SLM_API int slm_window_append(const slm_window_append_args* a, void* 
   if (a->rows == 0) return SLM_OK;
   const dim3 grid((unsigned)a->rows, (unsigned)((a->heads + 2 * a->kv_heads + 3) / 4));
   hip_clear_error();
-  if (a->dtype == SLM_BF16) window_append_kernel<bf16><<<grid, dim3(256), 0, (hipStream_t)stream>>>(*a);
-  else window_append_kernel<float><<<grid, dim3(256), 0, (hipStream_t)stream>>>(*a);
+  if (a->dtype == SLM_BF16) append_launch<bf16>(*a, grid, (hipStream_t)stream);
+  else append_launch<float>(*a, grid, (hipStream_t)stream);
   return hip_check_launch();
 }
 
