@@ -256,8 +256,11 @@ __global__ void __launch_bounds__(1024) recurrent_step_kernel(const slm_recurren
 //   S1 = diag(exp(L_end)) S0 + Kr^T U                 Kr_t = k_t exp(L_end - L_t)
 // Every exponent is <= 0: nothing overflows however fast a channel forgets.  Without the delta rule U = V.
 // A chunk's record for one head, in floats:
-//   Kd [16][DK] | Qd [16][DK] | Kr^T [DK][16] | exp(L_end) [DK] | V [16][v_pad] | T = (I + diag(beta) A)^-1 diag(beta) [16][16]
-//   | B [16][16]
+//   Kd | Qd (16 x DK each) | Kr^T (DK x 16) | exp(L_end) (DK) | V^T (v_pad x 16) | T = (I + diag(beta) A)^-1 diag(beta) | B (16 x 16)
+// Matrices are tiles of 16 x 16 in the order the scan's lanes take them, four floats a lane: entry (m, k) at
+// tile_at(m, k), so that a wave reads a tile as 1 KiB in a row.  Kd, Qd: m token, k channel; Kr^T, V^T: m channel / column,
+// k token; T, B: m row, k column.
+__device__ __forceinline__ int tile_at(int m, int k) { return (((k >> 2) & 3) * 16 + (m & 15)) * 4 + (k & 3); }
 template <int DK>
 struct ChunkRecord {
   static constexpr int KD = 0, QD = 16 * DK, KR = 32 * DK, GE = 48 * DK, V = 49 * DK;
@@ -304,8 +307,12 @@ __global__ void __launch_bounds__(256) recurrent_prepare_kernel(const slm_recurr
         }
       } else {
         const int c = i - 2 * DK;
-        float* dst = rec + ChunkRecord<DK>::V + c;
-        auto put = [&](int t, float x) { dst[t * a.v_pad] = x; };
+        float* dst = rec + ChunkRecord<DK>::V + (c >> 4) * 256 + (c & 15) * 4;
+        f32x4 four;
+        auto put = [&](int t, float x) {
+          four[t & 3] = x;
+          if ((t & 3) == 3) *reinterpret_cast<f32x4*>(dst + (t >> 2) * 64) = four;
+        };
         if (c < a.vdim) {
           conv_run4<E>(a, ring, row, row0, p, n, 2 * qk + head * a.vdim + c, put);
         } else {
@@ -329,8 +336,8 @@ __global__ void __launch_bounds__(256) recurrent_prepare_kernel(const slm_recurr
       }
       sq[t * LD + c] = q, sk[t * LD + c] = k;
     }
-    for (int i = tid; i < 16 * a.v_pad; i += 256) {
-      const int t = i / a.v_pad, c = i % a.v_pad;
+    for (int i = tid; i < 16 * a.v_pad; i += 256) {   // (in the record's order)
+      const int t = ((i >> 6) & 3) * 4 + (i & 3), c = (i >> 8) * 16 + ((i >> 2) & 15);
       float v = 0.f;
       if (t < n && c < a.vdim) {
         if constexpr (DELTA) v = conv_input<E>(a, ring, row + t, row0, p + t, 2 * qk + head * a.vdim + c);
@@ -399,20 +406,23 @@ __global__ void __launch_bounds__(256) recurrent_prepare_kernel(const slm_recurr
         y *= fast_exp2(sL[t * LD] - sL[s * LD]);
       }
     }
-    rec[at.b() + tid] = y;
+    rec[at.b() + tile_at(t, s)] = y;
     sa[t][s] = x;
   }
-  for (int i = 4 * tid; i < 16 * DK; i += 1024) {
-    const int t = i / DK, c = i % DK;
-    const f32x4 l = *reinterpret_cast<const f32x4*>(sL + t * LD + c), q = *reinterpret_cast<const f32x4*>(sq + t * LD + c);
-    const f32x4 e = {fast_exp2(l.x), fast_exp2(l.y), fast_exp2(l.z), fast_exp2(l.w)};
-    if constexpr (DELTA) *reinterpret_cast<f32x4*>(rec + ChunkRecord<DK>::KD + i) = *reinterpret_cast<const f32x4*>(sk + t * LD + c) * e;
-    *reinterpret_cast<f32x4*>(rec + ChunkRecord<DK>::QD + i) = q * e;
-    const int u = i & 15, d = i >> 4;
+  for (int i = tid; i < 4 * DK; i += 256) {   // four floats each, in the record's order
+    const int tile = i >> 6, m = i & 15, k = ((i >> 4) & 3) * 4;
+    {
+      const int at_t = m * LD + 16 * tile + k;
+      const f32x4 l = *reinterpret_cast<const f32x4*>(sL + at_t), q = *reinterpret_cast<const f32x4*>(sq + at_t);
+      const f32x4 e = {fast_exp2(l.x), fast_exp2(l.y), fast_exp2(l.z), fast_exp2(l.w)};
+      if constexpr (DELTA) *reinterpret_cast<f32x4*>(rec + ChunkRecord<DK>::KD + 4 * i) = *reinterpret_cast<const f32x4*>(sk + at_t) * e;
+      *reinterpret_cast<f32x4*>(rec + ChunkRecord<DK>::QD + 4 * i) = q * e;
+    }
+    const int d = 16 * tile + m;
     f32x4 kr;
 #pragma unroll
-    for (int j = 0; j < 4; ++j) kr[j] = sk[(u + j) * LD + d] * fast_exp2(sL[15 * LD + d] - sL[(u + j) * LD + d]);
-    *reinterpret_cast<f32x4*>(rec + ChunkRecord<DK>::KR + i) = kr;
+    for (int j = 0; j < 4; ++j) kr[j] = sk[(k + j) * LD + d] * fast_exp2(sL[15 * LD + d] - sL[(k + j) * LD + d]);
+    *reinterpret_cast<f32x4*>(rec + ChunkRecord<DK>::KR + 4 * i) = kr;
   }
   if (tid < DK) rec[ChunkRecord<DK>::GE + tid] = fast_exp2(sL[15 * LD + tid]);
   if constexpr (DELTA) {
@@ -425,32 +435,32 @@ __global__ void __launch_bounds__(256) recurrent_prepare_kernel(const slm_recurr
 #pragma unroll
         for (int s = 0; s < t; ++s) v = __builtin_fmaf(-sa[t][s], x[s], v);
         x[t] = sbeta[t] * v;
-        rec[at.t() + 16 * t + tid] = x[t];
+        rec[at.t() + tile_at(t, tid)] = x[t];
       }
     }
   }
 }
 
-// One workgroup per (sequence, head, 16 columns of S), chunk after chunk.  Its waves share the key channels: a wave keeps
-// TPW tiles [16 x 16] of S in registers in the accumulator layout of the 32-bit MFMA (row 4 g + r, column l16), which is the
-// layout its right operand takes when the contraction index of product r is 4 g + r.  Partial products with S0 meet in
-// LDS, one barrier a chunk; U is computed by every wave.  The operands of the next chunks
-// travel meanwhile.
-template <int TPW>
+// One workgroup per (sequence, head, 16 NCT columns of S), chunk after chunk.  Its waves share the key channels: a wave
+// keeps TPW tiles [16 x 16] of every column tile of S in registers in the accumulator layout of the 32-bit MFMA (row 4 g + r,
+// column l16), which is the layout its right operand takes when the contraction index of product r is 4 g + r.  Partial
+// products with S0 meet in LDS, one barrier a chunk; U is computed by every wave.  The operands of the next chunks travel
+// meanwhile.  Two column tiles read the records half as often: where enough workgroups are left.
+template <int TPW, int NCT>
 struct ChunkOperands {
-  f32x4 kd[TPW], qd[TPW], kr[TPW], ge[TPW], t, b, v;
+  f32x4 kd[TPW], qd[TPW], kr[TPW], ge[TPW], t, b, v[NCT];
 };
 
-template <typename E, int MODE, int DK, int W>
+template <typename E, int MODE, int DK, int W, int NCT>
 __global__ void __launch_bounds__(64 * W, 2) recurrent_scan_kernel(const slm_recurrent_args a) {
   constexpr bool DELTA = DELTA_MODE(MODE);
   constexpr int TPW = DK / 16 / W;
   constexpr int NB = TPW <= 2 ? 3 : 2;   // chunks in registers: one in use, the others on their way
-  __shared__ f32x4 part[2][2][W][64];
+  __shared__ f32x4 part[2][2][NCT][W][64];
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int l16 = lane & 15, g = lane >> 4;
   // the column blocks of one head on one XCD (workgroups go round the XCDs): they read the same records
-  const int n_cb = a.v_pad / 16, n_items = (a.batch - a.n_single) * a.heads;
+  const int n_ct = a.v_pad / 16, n_cb = (n_ct + NCT - 1) / NCT, n_items = (a.batch - a.n_single) * a.heads;
   const int cb = blockIdx.x / 8 % n_cb, item = blockIdx.x / (8 * n_cb) * 8 + blockIdx.x % 8;
   if (item >= n_items) return;
   const int head = item % a.heads, ps = item / a.heads, seq = a.n_single + ps;
@@ -462,66 +472,90 @@ __global__ void __launch_bounds__(64 * W, 2) recurrent_scan_kernel(const slm_rec
   const ChunkRecord<DK> at{a.v_pad};
   const float* rec0 = a.pre + (chunk0 * a.heads + head) * at.size();
   const int64_t rec_step = a.heads * at.size();
-  float* S = a.state + (((int64_t)slot * a.heads + head) * DK + 16 * TPW * wave + 4 * g) * a.v_pad + 16 * cb + l16;
-
-  f32x4 s[TPW];
+  float* S = a.state + (((int64_t)slot * a.heads + head) * DK + 16 * TPW * wave + 4 * g) * a.v_pad + l16;
+  int ct[NCT];   // (an odd last tile is computed twice and stored once)
 #pragma unroll
-  for (int i = 0; i < TPW; ++i)
-#pragma unroll
-    for (int r = 0; r < 4; ++r) s[i][r] = p0 > 0 ? S[(int64_t)(16 * i + r) * a.v_pad] : 0.f;
+  for (int j = 0; j < NCT; ++j) ct[j] = min(cb * NCT + j, n_ct - 1);
 
-  auto load = [&](int c, ChunkOperands<TPW>& x) {
+  f32x4 s[NCT][TPW];
+#pragma unroll
+  for (int j = 0; j < NCT; ++j)
+#pragma unroll
+    for (int i = 0; i < TPW; ++i)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) s[j][i][r] = p0 > 0 ? S[(int64_t)(16 * i + r) * a.v_pad + 16 * ct[j]] : 0.f;
+
+  // uniform bases and 32-bit lane offsets: an address is one register
+  auto vec = [](const float* base, uint32_t off) { return *reinterpret_cast<const f32x4*>(reinterpret_cast<const char*>(base) + off); };
+  const uint32_t off = (uint32_t)lane * 16, ge_off = (uint32_t)g * 16;
+  auto load = [&](int c, ChunkOperands<TPW, NCT>& x) {
     const float* rec = rec0 + c * rec_step;
 #pragma unroll
     for (int i = 0; i < TPW; ++i) {
-      const int d = 16 * (TPW * wave + i);
-      if constexpr (DELTA) x.kd[i] = *reinterpret_cast<const f32x4*>(rec + ChunkRecord<DK>::KD + l16 * DK + d + 4 * g);
-      x.qd[i] = *reinterpret_cast<const f32x4*>(rec + ChunkRecord<DK>::QD + l16 * DK + d + 4 * g);
-      x.kr[i] = *reinterpret_cast<const f32x4*>(rec + ChunkRecord<DK>::KR + (d + l16) * 16 + 4 * g);
-      x.ge[i] = *reinterpret_cast<const f32x4*>(rec + ChunkRecord<DK>::GE + d + 4 * g);
+      const int tile = TPW * wave + i;
+      if constexpr (DELTA) x.kd[i] = vec(rec + ChunkRecord<DK>::KD + 256 * tile, off);
+      x.qd[i] = vec(rec + ChunkRecord<DK>::QD + 256 * tile, off);
+      x.kr[i] = vec(rec + ChunkRecord<DK>::KR + 256 * tile, off);
+      x.ge[i] = vec(rec + ChunkRecord<DK>::GE + 16 * tile, ge_off);
     }
-    if constexpr (DELTA) x.t = *reinterpret_cast<const f32x4*>(rec + at.t() + l16 * 16 + 4 * g);
-    x.b = *reinterpret_cast<const f32x4*>(rec + at.b() + l16 * 16 + 4 * g);
+    if constexpr (DELTA) x.t = vec(rec + at.t(), off);
+    x.b = vec(rec + at.b(), off);
 #pragma unroll
-    for (int r = 0; r < 4; ++r) x.v[r] = rec[ChunkRecord<DK>::V + (4 * g + r) * a.v_pad + 16 * cb + l16];
+    for (int j = 0; j < NCT; ++j) x.v[j] = vec(rec + ChunkRecord<DK>::V + 256 * ct[j], off);
   };
   auto mma4 = [](const f32x4& x, const f32x4& y, f32x4 c) {
 #pragma unroll
     for (int r = 0; r < 4; ++r) c = __builtin_amdgcn_mfma_f32_16x16x4f32(x[r], y[r], c, 0, 0, 0);
     return c;
   };
-  auto chunk = [&](int c, const ChunkOperands<TPW>& x) {
+  auto chunk = [&](int c, const ChunkOperands<TPW, NCT>& x) {
     const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
     const int b = c & 1;
-    f32x4 kr = zero, o = zero;
+    f32x4 kr[NCT], o[NCT], u[NCT];
 #pragma unroll
-    for (int i = 0; i < TPW; ++i) {
-      if constexpr (DELTA) kr = mma4(x.kd[i], s[i], kr);
-      o = mma4(x.qd[i], s[i], o);
+    for (int j = 0; j < NCT; ++j) kr[j] = o[j] = zero;
+#pragma unroll
+    for (int i = 0; i < TPW; ++i)
+#pragma unroll
+      for (int j = 0; j < NCT; ++j) {
+        if constexpr (DELTA) kr[j] = mma4(x.kd[i], s[j][i], kr[j]);
+        o[j] = mma4(x.qd[i], s[j][i], o[j]);
+      }
+#pragma unroll
+    for (int j = 0; j < NCT; ++j) {
+      if constexpr (DELTA) part[b][0][j][wave][lane] = kr[j];
+      part[b][1][j][wave][lane] = o[j];
     }
-    if constexpr (DELTA) part[b][0][wave][lane] = kr;
-    part[b][1][wave][lane] = o;
     lds_barrier();
-    f32x4 u = x.v;
-    if constexpr (DELTA) {
 #pragma unroll
-      for (int w = 0; w < W; ++w) u -= part[b][0][w][lane];
-      u = mma4(x.t, u, zero);
+    for (int j = 0; j < NCT; ++j) {
+      u[j] = x.v[j];
+      if constexpr (DELTA) {
+#pragma unroll
+        for (int w = 0; w < W; ++w) u[j] -= part[b][0][j][w][lane];
+        u[j] = mma4(x.t, u[j], zero);
+      }
     }
 #pragma unroll
-    for (int i = 0; i < TPW; ++i) s[i] = mma4(x.kr[i], u, s[i] * x.ge[i]);
-    if (c % W == wave) {   // (the waves take the outputs in turn)
-      o = part[b][1][0][lane];
+    for (int i = 0; i < TPW; ++i)
 #pragma unroll
-      for (int w = 1; w < W; ++w) o += part[b][1][w][lane];
-      o = mma4(x.b, u, o);
-      float* dst = a.o + ((row0 - a.n_single + 16 * c + 4 * g) * a.heads + head) * a.v_pad + 16 * cb + l16;
+      for (int j = 0; j < NCT; ++j) s[j][i] = mma4(x.kr[i], u[j], s[j][i] * x.ge[i]);
 #pragma unroll
-      for (int r = 0; r < 4; ++r)
-        if (16 * c + 4 * g + r < n) dst[(int64_t)r * a.heads * a.v_pad] = o[r];
-    }
+    for (int j = 0; j < NCT; ++j)
+      if ((c * NCT + j) % W == wave && cb * NCT + j < n_ct) {   // (the waves take the outputs in turn)
+        f32x4 y = part[b][1][j][0][lane];
+#pragma unroll
+        for (int w = 1; w < W; ++w) y += part[b][1][j][w][lane];
+        y = mma4(x.b, u[j], y);
+        float* dst = a.o + ((row0 - a.n_single + 16 * c) * a.heads + head) * a.v_pad + 16 * ct[j];
+        const uint32_t o_off = (uint32_t)(4 * g * a.heads * a.v_pad + l16) * 4;
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          if (16 * c + 4 * g + r < n)
+            *reinterpret_cast<float*>(reinterpret_cast<char*>(dst + (int64_t)r * a.heads * a.v_pad) + o_off) = y[r];
+      }
   };
-  ChunkOperands<TPW> x[NB];
+  ChunkOperands<TPW, NCT> x[NB];
 #pragma unroll
   for (int i = 0; i + 1 < NB; ++i) load(min(i, n_chunks - 1), x[i]);
   int c0 = 0;   // (whole rounds without a branch around the loads: a join would make every wait one for the youngest)
@@ -536,9 +570,12 @@ __global__ void __launch_bounds__(64 * W, 2) recurrent_scan_kernel(const slm_rec
   for (int i = 0; i + 1 < NB; ++i)
     if (c0 + i < n_chunks) chunk(c0 + i, x[i]);
 #pragma unroll
-  for (int i = 0; i < TPW; ++i)
+  for (int j = 0; j < NCT; ++j)
+    if (cb * NCT + j < n_ct)
 #pragma unroll
-    for (int r = 0; r < 4; ++r) S[(int64_t)(16 * i + r) * a.v_pad] = s[i][r];
+      for (int i = 0; i < TPW; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) S[(int64_t)(16 * i + r) * a.v_pad + 16 * ct[j]] = s[j][i][r];
 
   // the last inputs of the convolutions (their readers ran in the launch before)
   if (DELTA && cb == 0) {
@@ -606,6 +643,7 @@ __global__ void __launch_bounds__(256) gated_norm_kernel(const slm_gated_norm_ar
   }
 }
 
+constexpr int64_t NCT2_MIN = 512;   // column tiles from which a workgroup takes two
 static bool rec_sizes_ok(const slm_recurrent_args& a) {
   return a.heads > 0 && a.qk_heads > 0 && a.heads % a.qk_heads == 0 && a.dim > 0 && a.vdim > 0 && a.vdim <= a.v_pad &&
          a.v_pad % 16 == 0 && a.v_pad <= 256 && a.dim_pad >= a.dim && a.dim_pad == slm_recurrent_dim_pad(a.dim) &&
@@ -631,11 +669,16 @@ static int rec_step(const slm_recurrent_args& a, hipStream_t st) {
   }
   return hip_check_launch();
 }
+template <typename E, int MODE, int DK, int NCT>
+static void rec_scan_nct(const slm_recurrent_args& a, hipStream_t st) {
+  constexpr int W = DK / 16 < 4 ? DK / 16 : 4;
+  const int64_t items = (int64_t)(a.batch - a.n_single) * a.heads, n_cb = (a.v_pad / 16 + NCT - 1) / NCT;
+  recurrent_scan_kernel<E, MODE, DK, W, NCT><<<dim3((unsigned)((items + 7) / 8 * 8 * n_cb)), dim3(64 * W), 0, st>>>(a);
+}
 template <typename E, int MODE, int DK>
 static void rec_scan_dk(const slm_recurrent_args& a, hipStream_t st) {
-  constexpr int W = DK / 16 < 4 ? DK / 16 : 4;
-  const int64_t items = (int64_t)(a.batch - a.n_single) * a.heads;
-  recurrent_scan_kernel<E, MODE, DK, W><<<dim3((unsigned)((items + 7) / 8 * 8 * (a.v_pad / 16))), dim3(64 * W), 0, st>>>(a);
+  if (DK <= 128 && (int64_t)(a.batch - a.n_single) * a.heads * (a.v_pad / 16) >= NCT2_MIN) rec_scan_nct<E, MODE, DK, (DK <= 128 ? 2 : 1)>(a, st);
+  else rec_scan_nct<E, MODE, DK, 1>(a, st);
 }
 template <typename E, int MODE>
 static int rec_scan(const slm_recurrent_args& a, hipStream_t st) {

@@ -48,7 +48,7 @@ def _parse_mixer(i: int, e: dict):
     if e["type"] != "parallel":
         raise ValueError(f"layer {i}: unknown mixer {e['type']!r}")
     a, b = m["left"], m["right"]
-    rot, mask = a["rot"], a.get("mask") or {}
+    rot, mask = a.get("rot") or {"base": 1.0, "dims": 0}, a.get("mask") or {}
     if rot["dims"] % 2 or rot["dims"] > a["dim"]:
         raise ValueError(f"layer {i}: {rot['dims']} rotated dimensions of {a['dim']}")
     left = WindowAttentionArgs(heads=a["heads"], kv_heads=a["kv_heads"], dim=a["dim"], vdim=a["vdim"], scale=a["scale"],
@@ -110,7 +110,7 @@ class VebusunStep:
         f32 = lambda name: ckpt.take(name, (W,)).to(device=dev, dtype=torch.float32).contiguous()  # noqa: E731
 
         def norm(name):
-            return lk.TanhNorm(ckpt.take(name + ".alpha", ()).float().item(), f32(name), f32(name + ".b"))
+            return lk.TanhNorm(ckpt.take(name + ".alpha").float().item(), f32(name), f32(name + ".b"))   # (a scalar)
         self.final_norm = norm("final.norm")
         tables = {}
 
@@ -130,6 +130,8 @@ class VebusunStep:
                 L.mlp = ClampedGLU(W, layer.ff, math.inf, {"gate": ckpt.take(p + "mlp.gate", (layer.ff, W)),
                                                            "up": ckpt.take(p + "mlp.up", (layer.ff, W)),
                                                            "down": ckpt.take(p + "mlp.down", (W, layer.ff))}, dt, dev, 1.0, 0.0)
+            elif p + "norm2" in ckpt.names():   # (a norm nothing follows)
+                norm(p + "norm2")
             weights.append(L)
         self.layers = [weights[i] for i in c.runs]
         self.caches = [L.mixer.new_cache(limits) for L in self.layers]
