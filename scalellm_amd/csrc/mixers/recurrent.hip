@@ -444,7 +444,7 @@ __global__ void __launch_bounds__(256) recurrent_prepare_kernel(const slm_recurr
 // One workgroup per (sequence, head, 16 NCT columns of S), chunk after chunk.  Its waves share the key channels: a wave
 // keeps TPW tiles [16 x 16] of every column tile of S in registers in the accumulator layout of the 32-bit MFMA (row 4 g + r,
 // column l16), which is the layout its right operand takes when the contraction index of product r is 4 g + r.  Partial
-// products with S0 meet in LDS, one barrier a chunk; U is computed by every wave.  The operands of the next chunks travel
+// products with S0 meet in LDS, one barrier a chunk; U is computed by every wave; read-outs are completed a chunk later.  The operands of the next chunks travel
 // meanwhile.  Two column tiles read the records half as often: where enough workgroups are left.
 template <int TPW, int NCT>
 struct ChunkOperands {
@@ -455,8 +455,8 @@ template <typename E, int MODE, int DK, int W, int NCT>
 __global__ void __launch_bounds__(64 * W, 2) recurrent_scan_kernel(const slm_recurrent_args a) {
   constexpr bool DELTA = DELTA_MODE(MODE);
   constexpr int TPW = DK / 16 / W;
-  constexpr int NB = TPW <= 2 ? 3 : 2;   // chunks in registers: one in use, the others on their way
-  __shared__ f32x4 part[2][2][NCT][W][64];
+  constexpr int NB = TPW <= (DELTA ? 1 : 2) ? 3 : 2;   // chunks in registers: one in use, the others on their way
+  __shared__ f32x4 part_u[2][NCT][W][64], part_o[2][NCT][W][64];
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int l16 = lane & 15, g = lane >> 4;
   // the column blocks of one head on one XCD (workgroups go round the XCDs): they read the same records
@@ -508,31 +508,47 @@ __global__ void __launch_bounds__(64 * W, 2) recurrent_scan_kernel(const slm_rec
     for (int r = 0; r < 4; ++r) c = __builtin_amdgcn_mfma_f32_16x16x4f32(x[r], y[r], c, 0, 0, 0);
     return c;
   };
+  auto finish = [&](int c) {   // the read-outs of chunk c, once every wave's part of them is there
+#pragma unroll
+    for (int j = 0; j < NCT; ++j)
+      if ((c * NCT + j + W / 2) % W == wave && cb * NCT + j < n_ct) {
+        f32x4 y = part_o[c & 1][j][0][lane];
+#pragma unroll
+        for (int w = 1; w < W; ++w) y += part_o[c & 1][j][w][lane];
+        float* dst = a.o + ((row0 - a.n_single + 16 * c) * a.heads + head) * a.v_pad + 16 * ct[j];
+        const uint32_t o_off = (uint32_t)(4 * g * a.heads * a.v_pad + l16) * 4;
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          if (16 * c + 4 * g + r < n)
+            *reinterpret_cast<float*>(reinterpret_cast<char*>(dst + (int64_t)r * a.heads * a.v_pad) + o_off) = y[r];
+      }
+  };
   auto chunk = [&](int c, const ChunkOperands<TPW, NCT>& x) {
     const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
     const int b = c & 1;
     f32x4 kr[NCT], o[NCT], u[NCT];
 #pragma unroll
     for (int j = 0; j < NCT; ++j) kr[j] = o[j] = zero;
+    if constexpr (DELTA) {
+#pragma unroll
+      for (int i = 0; i < TPW; ++i)
+#pragma unroll
+        for (int j = 0; j < NCT; ++j) kr[j] = mma4(x.kd[i], s[j][i], kr[j]);
+#pragma unroll
+      for (int j = 0; j < NCT; ++j) part_u[b][j][wave][lane] = kr[j];
+    }
+    // (what the next chunk does not wait for runs under the exchange)
 #pragma unroll
     for (int i = 0; i < TPW; ++i)
 #pragma unroll
-      for (int j = 0; j < NCT; ++j) {
-        if constexpr (DELTA) kr[j] = mma4(x.kd[i], s[j][i], kr[j]);
-        o[j] = mma4(x.qd[i], s[j][i], o[j]);
-      }
-#pragma unroll
-    for (int j = 0; j < NCT; ++j) {
-      if constexpr (DELTA) part[b][0][j][wave][lane] = kr[j];
-      part[b][1][j][wave][lane] = o[j];
-    }
+      for (int j = 0; j < NCT; ++j) o[j] = mma4(x.qd[i], s[j][i], o[j]);
     lds_barrier();
 #pragma unroll
     for (int j = 0; j < NCT; ++j) {
       u[j] = x.v[j];
       if constexpr (DELTA) {
 #pragma unroll
-        for (int w = 0; w < W; ++w) u[j] -= part[b][0][j][w][lane];
+        for (int w = 0; w < W; ++w) u[j] -= part_u[b][j][w][lane];
         u[j] = mma4(x.t, u[j], zero);
       }
     }
@@ -541,19 +557,11 @@ __global__ void __launch_bounds__(64 * W, 2) recurrent_scan_kernel(const slm_rec
 #pragma unroll
       for (int j = 0; j < NCT; ++j) s[j][i] = mma4(x.kr[i], u[j], s[j][i] * x.ge[i]);
 #pragma unroll
-    for (int j = 0; j < NCT; ++j)
-      if ((c * NCT + j) % W == wave && cb * NCT + j < n_ct) {   // (the waves take the outputs in turn)
-        f32x4 y = part[b][1][j][0][lane];
-#pragma unroll
-        for (int w = 1; w < W; ++w) y += part[b][1][j][w][lane];
-        y = mma4(x.b, u[j], y);
-        float* dst = a.o + ((row0 - a.n_single + 16 * c) * a.heads + head) * a.v_pad + 16 * ct[j];
-        const uint32_t o_off = (uint32_t)(4 * g * a.heads * a.v_pad + l16) * 4;
-#pragma unroll
-        for (int r = 0; r < 4; ++r)
-          if (16 * c + 4 * g + r < n)
-            *reinterpret_cast<float*>(reinterpret_cast<char*>(dst + (int64_t)r * a.heads * a.v_pad) + o_off) = y[r];
-      }
+    for (int j = 0; j < NCT; ++j) {   // (the waves take B U, and the stores a barrier later, in turn)
+      if ((c * NCT + j) % W == wave) o[j] = mma4(x.b, u[j], o[j]);
+      part_o[b][j][wave][lane] = o[j];
+    }
+    if (c > 0) finish(c - 1);
   };
   ChunkOperands<TPW, NCT> x[NB];
 #pragma unroll
@@ -569,6 +577,8 @@ __global__ void __launch_bounds__(64 * W, 2) recurrent_scan_kernel(const slm_rec
 #pragma unroll
   for (int i = 0; i + 1 < NB; ++i)
     if (c0 + i < n_chunks) chunk(c0 + i, x[i]);
+  lds_barrier();
+  finish(n_chunks - 1);
 #pragma unroll
   for (int j = 0; j < NCT; ++j)
     if (cb * NCT + j < n_ct)
