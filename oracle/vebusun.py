@@ -1,5 +1,5 @@
 """Plain, slow restatement of the Vebusun design in double precision (numpy): one function per mechanism, no cache, no
-batch, no padding, one token after the other where a recurrence runs.  Checker only; shares no code with scalellm_amd."""
+batch, no padding, one token after the other where a recurrence runs.  For tests only; shares no code with scalellm_amd."""
 from __future__ import annotations
 
 import numpy as np
